@@ -204,7 +204,10 @@ class BenaraxLatentAttention(nn.Module, _FusedInputs):
         return PagedKVSpec(1, self.m.kv_rank + self.m.rot_dim, self.m.kv_rank, value_in_key=True)
 
     def finalize(self):
+        m = self.m
         self._fuse(self._inputs)
+        # a bfloat16 batched product takes a contiguous right operand only (a transposed view of one can fault the GPU)
+        self._uv_t = self.uv.weight.data.view(m.heads, m.vdim, m.kv_rank).transpose(1, 2).contiguous()
 
     def forward(self, x, positions, cache):
         m, H = self.m, self.m.heads
@@ -214,7 +217,7 @@ class BenaraxLatentAttention(nn.Module, _FusedInputs):
         q_lat = torch.bmm(q[:, :, :m.dim].transpose(0, 1), self.uk.weight.view(H, m.dim, m.kv_rank))      # [H, T, rank]
         o_lat = self.attn(q, q_lat.transpose(0, 1), ckv, positions, cache[0], cache[1])                   # [T, H, rank]
         # ... and the value up-projection to the output
-        o = torch.bmm(o_lat.transpose(0, 1), self.uv.weight.view(H, m.vdim, m.kv_rank).transpose(1, 2))   # [H, T, vdim]
+        o = torch.bmm(o_lat.transpose(0, 1), self._uv_t)                                                  # [H, T, vdim]
         return self.o(o.transpose(0, 1).reshape(x.shape[0], H * m.vdim))
 
 

@@ -259,9 +259,11 @@ class DivadraTimeMix(nn.Module):
         if self.w2.weight.shape[1] != self.w1.weight.shape[0]:
             raise ValueError("low-rank decay projections do not chain")
         # r, k, v, g read different blends: one batched product over the stacked weights (the Linear weights become views)
-        w = torch.stack([getattr(self, n).weight.data for n in ("r", "k", "v", "g")])
+        # (stored transposed: a bfloat16 batched product takes a contiguous right operand only, a transposed view can fault
+        # the GPU)
+        w = torch.stack([getattr(self, n).weight.data.t() for n in ("r", "k", "v", "g")])
         for i, n in enumerate(("r", "k", "v", "g")):
-            getattr(self, n).weight.data = w[i]
+            getattr(self, n).weight.data = w[i].t()
         self._stacked = w
 
     def forward(self, h, positions, cache):
@@ -269,7 +271,7 @@ class DivadraTimeMix(nn.Module):
         mixes = self.shift(h, cache["prev"])                                      # [5, T, W]
         w = self._stacked
         if w is not None and w.device == h.device and w.dtype == h.dtype:
-            r, k, v, g = torch.bmm(mixes[:4], w.transpose(1, 2)).unbind(0)
+            r, k, v, g = torch.bmm(mixes[:4], w).unbind(0)
         else:
             r, k, v, g = (getattr(self, n)(mixes[i]) for i, n in enumerate(("r", "k", "v", "g")))
         w_raw = self.w2(torch.tanh(self.w1(mixes[4]).float()).to(h.dtype))
