@@ -399,6 +399,45 @@ NV_API int nv_moe_up_relu2(const void* h, int64_t h_stride, const void* up, cons
                            const int32_t* meta, void* y, int dtype, int64_t pairs, int E, int top, int width, int ff,
                            int tile_rows, void* stream);
 
+/*
+ * Routing by softmax scores over all E experts: the choice is made on score + correction (NULL: the score), weights =
+ * scale * score of the chosen, not renormalised.  E <= 1024.  nv_moe_align leaves pairs out whose id is not below its E,
+ * so the last experts may be ones without a product (identity experts).
+ */
+NV_API int nv_moe_route_softmax(const float* logits, const float* correction, int32_t* ids, float* weights, int64_t T,
+                                int E, int top, float scale, void* stream);
+
+/* x[t] = embed[ids[t]] + pos[positions[t]] in fp32; embed [vocab, cols], pos [max_positions, cols] of dtype. */
+NV_API int nv_embed_positions(const int64_t* ids, const int64_t* positions, const void* embed, const void* pos, float* x,
+                              int dtype, int64_t T, int cols, int64_t vocab, int64_t max_positions, void* stream);
+
+/*
+ * One layer boundary of an fp32 residual stream that two parallel sublayers read, per row:
+ *   r <- r + add1 + add2 + sum over j with ids[j] < experts of parts[j] + (sum of weights[j], ids[j] >= experts) * through
+ *   y1 <- LN(r) * w1 + b1 (dtype);   y2 <- LN(r) * w2 + b2 (dtype and / or fp32)
+ * add1, add2, through: [rows, cols] of dtype with row strides; parts: [rows, n_parts, cols] fp32; ids / weights:
+ * [rows, n_parts] (NULL: every part counts).  Each of add1, add2, parts, through and the two norms may be NULL.
+ */
+NV_API int nv_stream_layernorm_pair(float* resid, const void* add1, int64_t add1_stride, const void* add2,
+                                    int64_t add2_stride, const float* parts, const int32_t* ids, const float* weights,
+                                    int n_parts, int experts, const void* through, int64_t through_stride,
+                                    const float* w1, const float* b1, const float* w2, const float* b2, float eps,
+                                    void* y1, void* y2, float* y2_f32, int dtype, int64_t rows, int cols, void* stream);
+
+/* y[r, j] = silu(x[r, j]) * x[r, inter + j], any inter, bf16 or fp32. */
+NV_API int nv_silu_and_mul_rows(const void* x, int64_t x_stride, void* y, int dtype, int64_t rows, int inter,
+                                void* stream);
+
+/* cache[slot_mapping[t]] = ckv[t] / sqrt(mean(ckv[t]^2) + eps) * latent_w, rows of `rank`; slots outside 0 .. num_slots - 1
+ * are skipped. */
+NV_API int nv_latent_store(const void* ckv, int64_t ckv_stride, const float* latent_w, const int32_t* slot_mapping,
+                           void* cache, int64_t num_slots, int dtype, int64_t T, int rank, float eps, void* stream);
+
+/* y[t, h, n] = sum_k x[t, h, k] * w[h, n, k], times sigmoid(gate[t, h * N + n]) if gate; x: [T, H, K] with a token stride
+ * (heads contiguous), w: [H, N, K], gate: [T, H * N] with a row stride, y: [T, H, N] contiguous. */
+NV_API int nv_head_linear(const void* x, int64_t x_stride, const void* w, const void* gate, int64_t gate_stride, void* y,
+                          int dtype, int64_t T, int H, int N, int K, void* stream);
+
 #ifdef __cplusplus
 }
 #endif

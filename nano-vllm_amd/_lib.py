@@ -12,7 +12,7 @@ import threading
 _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_HERE, "lib", "libnanovllm_hip.so")
 MIXERS_LIB_PATH = os.path.join(_HERE, "lib", "libnanovllm_hip_mixers.so")
-ABI_VERSION = 11
+ABI_VERSION = 12
 
 _vp, _i32, _i64, _f32 = C.c_void_p, C.c_int, C.c_int64, C.c_float
 
@@ -128,6 +128,13 @@ MIXERS_PROTOTYPES = {
     "nv_gated_write_memory": (_i32, [_vp, _vp, _vp, _i64, _i64, _i64, _vp, _vp, _vp, _vp, _vp, _i64, _vp, _vp, _vp, _i32,
                                      _i32, _i32, _i32, _f32, _i32, _vp]),
     "nv_moe_route_grouped": (_i32, [_vp, _vp, _vp, _vp, _i64, _i32, _i32, _i32, _i32, _vp]),
+    "nv_moe_route_softmax": (_i32, [_vp, _vp, _vp, _vp, _i64, _i32, _i32, _f32, _vp]),
+    "nv_embed_positions": (_i32, [_vp, _vp, _vp, _vp, _vp, _i32, _i64, _i32, _i64, _i64, _vp]),
+    "nv_stream_layernorm_pair": (_i32, [_vp, _vp, _i64, _vp, _i64, _vp, _vp, _vp, _i32, _i32, _vp, _i64, _vp, _vp, _vp, _vp,
+                                        _f32, _vp, _vp, _vp, _i32, _i64, _i32, _vp]),
+    "nv_silu_and_mul_rows": (_i32, [_vp, _i64, _vp, _i32, _i64, _i32, _vp]),
+    "nv_latent_store": (_i32, [_vp, _i64, _vp, _vp, _vp, _i64, _i32, _i64, _i32, _f32, _vp]),
+    "nv_head_linear": (_i32, [_vp, _i64, _vp, _vp, _i64, _vp, _i32, _i64, _i32, _i32, _i32, _vp]),
     "nv_moe_up_relu2": (_i32, [_vp, _i64, _vp, _vp, _vp, _vp, _i32, _i64, _i32, _i32, _i32, _i32, _i32, _vp]),
 }
 DTYPE_BF16, DTYPE_F32 = 0, 1

@@ -2,6 +2,9 @@
 //
 // nv_moe_route          per token, from fp32 router logits [T, E]: the `top` largest (lowest index first among equals),
 //                       their weights = softmax over the chosen logits only.  ids [T, top] int32, weights [T, top] fp32.
+// nv_moe_route_softmax  the same shape of answer from softmax scores over ALL experts: the choice is made on score +
+//                       correction, the weights are the plain scores times a constant.  Ids beyond the experts that have
+//                       tensors (experts that hand their input through) are left out by nv_moe_align.
 // nv_moe_align          sorts the T * top (token, choice) pairs by expert: sorted_pairs[position] = pair index, and a
 //                       table of row tiles (expert, first position, rows) of at most `tile_rows` rows that never
 //                       straddle two experts, plus their count, all on the device.
@@ -18,7 +21,7 @@
 // routing can produce; workgroups beyond the table's count return at once.
 #include <algorithm>
 
-#include "nv_common.h"
+#include "mfma_tile.h"
 #include "../../include/nanovllm_hip_mixers.h"
 
 namespace nv {
@@ -145,7 +148,57 @@ __global__ __launch_bounds__(64) void moe_route_grouped_kernel(const float* __re
     }
 }
 
-// One workgroup.  meta: [0] = number of tiles, then (expert, first position, rows) per tile.
+// Softmax scores over all experts, a choice on score + correction, weights = scale * score of the chosen.  One wave per
+// token: scores and choice values live in LDS, each choice is a wave-wide arg-max (larger value, then lower index) after
+// which the winner's lane strikes it out.
+constexpr int kMoeSoftmaxMaxE = 1024;
+__global__ __launch_bounds__(64) void moe_route_softmax_kernel(const float* __restrict__ logits, const float* __restrict__ corr,
+                                                               int* __restrict__ ids, float* __restrict__ wgt, int E, int top,
+                                                               float scale) {
+    __shared__ float score[kMoeSoftmaxMaxE];
+    __shared__ float choice[kMoeSoftmaxMaxE];
+    const int64_t t = blockIdx.x;
+    const int lane = threadIdx.x;
+    const float* z = logits + t * E;
+    float zmax = -INFINITY;
+    for (int e = lane; e < E; e += 64) zmax = fmaxf(zmax, z[e]);
+#pragma unroll
+    for (int off = 32; off >= 1; off >>= 1) zmax = fmaxf(zmax, __shfl_xor(zmax, off));
+    float sum = 0.f;
+    for (int e = lane; e < E; e += 64) {
+        const float p = expf(z[e] - zmax);
+        score[e] = p;
+        sum += p;
+    }
+    const float inv = 1.0f / wave_sum(sum);
+    for (int e = lane; e < E; e += 64) {               // (a lane reads back what it wrote itself)
+        const float s = score[e] * inv;
+        score[e] = s;
+        choice[e] = corr != nullptr ? s + corr[e] : s;
+    }
+    __syncthreads();
+    unsigned taken = 0;                                // bit i: expert lane + 64 i is chosen
+    for (int j = 0; j < top; ++j) {
+        float bv = -INFINITY;
+        int be = E;                                    // E: nothing found
+        for (int i = 0, e = lane; e < E; ++i, e += 64)
+            if (!((taken >> i) & 1u) && (be == E || choice[e] > bv)) { bv = choice[e]; be = e; }
+#pragma unroll
+        for (int off = 32; off >= 1; off >>= 1) {
+            const float ov = __shfl_xor(bv, off);
+            const int oe = __shfl_xor(be, off);
+            if (oe < E && (be == E || ov > bv || (ov == bv && oe < be))) { bv = ov; be = oe; }
+        }
+        if ((be & 63) == lane) taken |= 1u << (be >> 6);
+        if (lane == 0) {
+            ids[t * top + j] = be;
+            wgt[t * top + j] = scale * score[be < E ? be : 0];
+        }
+    }
+}
+
+// One workgroup.  meta: [0] = number of tiles, then (expert, first position, rows) per tile.  A pair whose id is not in
+// 0 .. E - 1 (a choice that needs no product) gets no position.
 __global__ __launch_bounds__(1024) void moe_align_kernel(const int* __restrict__ ids, int* __restrict__ sorted_pairs,
                                                          int* __restrict__ meta, int64_t P, int E, int tile_rows) {
     extern __shared__ int sm[];                    // [E] counts, [E] cursors
@@ -154,7 +207,10 @@ __global__ __launch_bounds__(1024) void moe_align_kernel(const int* __restrict__
     const int tid = threadIdx.x;
     for (int e = tid; e < E; e += 1024) count[e] = 0;
     __syncthreads();
-    for (int64_t p = tid; p < P; p += 1024) atomicAdd(&count[ids[p]], 1);
+    for (int64_t p = tid; p < P; p += 1024) {
+        const int e = ids[p];
+        if (e >= 0 && e < E) atomicAdd(&count[e], 1);
+    }
     __syncthreads();
     if (tid == 0) {
         int off = 0, n = 0;
@@ -172,34 +228,10 @@ __global__ __launch_bounds__(1024) void moe_align_kernel(const int* __restrict__
         meta[0] = n;
     }
     __syncthreads();
-    for (int64_t p = tid; p < P; p += 1024) sorted_pairs[atomicAdd(&cursor[ids[p]], 1)] = (int)p;
-}
-
-template <typename T> struct MoeMma;
-template <> struct MoeMma<__bf16> {
-    static constexpr int kVec = 8, kPad = 8, kStep = 32, kBK = 64;
-    // the 32-deep product of gfx950: a lane holds 8 consecutive k of its row (16-byte LDS reads)
-    static __device__ __forceinline__ f32x4 run(const __bf16* a, const __bf16* b, int lg, f32x4 c) {
-        return __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)(a + 8 * lg), *(const bf16x8*)(b + 8 * lg), c, 0, 0, 0);
+    for (int64_t p = tid; p < P; p += 1024) {
+        const int e = ids[p];
+        if (e >= 0 && e < E) sorted_pairs[atomicAdd(&cursor[e], 1)] = (int)p;
     }
-};
-template <> struct MoeMma<float> {
-    static constexpr int kVec = 4, kPad = 4, kStep = 4, kBK = 32;
-    static __device__ __forceinline__ f32x4 run(const float* a, const float* b, int lg, f32x4 c) {
-        return __builtin_amdgcn_mfma_f32_16x16x4f32(a[lg], b[lg], c, 0, 0, 0);
-    }
-};
-
-// 16 bytes (kVec elements) of a row starting at k0, zeros past K or for a missing row
-template <typename T>
-__device__ __forceinline__ uint4 moe_fetch(const T* row, int k0, int K, bool vec_ok) {
-    constexpr int V = MoeMma<T>::kVec;
-    if (row == nullptr || k0 >= K) return make_uint4(0, 0, 0, 0);
-    if (vec_ok && k0 + V <= K) return *(const uint4*)(row + k0);
-    __attribute__((aligned(16))) T tmp[V];
-#pragma unroll
-    for (int i = 0; i < V; ++i) tmp[i] = k0 + i < K ? row[k0 + i] : (T)0.f;
-    return *(const uint4*)tmp;
 }
 
 // MODE 1 (gate and up): A rows are gathered token rows, B holds the expert's gate rows and up rows, the epilogue is the
@@ -212,7 +244,7 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(
     const T* __restrict__ a, int64_t a_stride, const T* __restrict__ w, const int* __restrict__ sorted_pairs,
     const int* __restrict__ meta, const float* __restrict__ pair_w, T* __restrict__ y, float* __restrict__ out, int top,
     int N, int K, float limit, float alpha, float up_shift, int vec_ok, int max_tiles) {
-    using M = MoeMma<T>;
+    using M = TileMma<T>;
     constexpr bool GATE_UP = MODE == 1, GATHER = MODE != 0;
     constexpr int BK = M::kBK, BM = 16 * MT, BN = 64 * NT, NB = GATE_UP ? 2 : 1, LD = BK + M::kPad, KV = BK / M::kVec;
     constexpr int A_IT = (BM * KV + 255) / 256, B_IT = (NB * BN * KV + 255) / 256;
@@ -252,9 +284,9 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(
     uint4 a_reg[A_IT], b_reg[B_IT];
     auto fetch = [&](int k0) {
 #pragma unroll
-        for (int i = 0; i < A_IT; ++i) a_reg[i] = moe_fetch<T>(a_row[i], k0 + ((tid + 256 * i) % KV) * M::kVec, K, vec_ok != 0);
+        for (int i = 0; i < A_IT; ++i) a_reg[i] = tile_fetch<T>(a_row[i], k0 + ((tid + 256 * i) % KV) * M::kVec, K, vec_ok != 0);
 #pragma unroll
-        for (int i = 0; i < B_IT; ++i) b_reg[i] = moe_fetch<T>(b_row[i], k0 + ((tid + 256 * i) % KV) * M::kVec, K, vec_ok != 0);
+        for (int i = 0; i < B_IT; ++i) b_reg[i] = tile_fetch<T>(b_row[i], k0 + ((tid + 256 * i) % KV) * M::kVec, K, vec_ok != 0);
     };
     f32x4 acc[NB * NT][MT];
 #pragma unroll
@@ -316,7 +348,7 @@ template <typename T, int MODE>
 static void launch_grouped(const void* a, int64_t a_stride, const void* w, const int* sorted_pairs, const int* meta,
                            const float* pair_w, void* y, float* out, int top, int N, int K, float limit, float alpha,
                            float up_shift, int max_tiles, int tile_rows, hipStream_t s) {
-    const int vec = MoeMma<T>::kVec;
+    const int vec = TileMma<T>::kVec;
     const int vec_ok = K % vec == 0 && a_stride % vec == 0 && ((uintptr_t)a | (uintptr_t)w) % 16 == 0;
     // many rows per expert: 64 x 128 tiles (a wave owns 32 columns; 128-row tiles measured slower: one workgroup per CU);
     // few: 16 x 64 tiles, more workgroups per weight byte
@@ -447,4 +479,18 @@ extern "C" int nv_moe_up_relu2(const void* h, int64_t h_stride, const void* up, 
         launch_grouped<float, 2>(h, h_stride, up, sorted_pairs, meta, nullptr, y, nullptr, top, ff, width, 0.f, 0.f, 0.f,
                                  (int)tiles, tile_rows, s);
     return check_launch("nv_moe_up_relu2");
+}
+
+extern "C" int nv_moe_route_softmax(const float* logits, const float* correction, int32_t* ids, float* weights, int64_t T,
+                                    int E, int top, float scale, void* stream) {
+    using namespace nv;
+    NV_REQUIRE(T >= 0 && E > 0 && E <= kMoeSoftmaxMaxE, NV_ERR_INVALID_ARG, "nv_moe_route_softmax: E=%d must lie in 1 .. %d",
+               E, kMoeSoftmaxMaxE);
+    NV_REQUIRE(top >= 1 && top <= E, NV_ERR_INVALID_ARG, "nv_moe_route_softmax: top=%d must lie in 1 .. E=%d", top, E);
+    if (T == 0) return NV_OK;
+    NV_REQUIRE(logits && ids && weights, NV_ERR_INVALID_ARG, "nv_moe_route_softmax: null pointer");
+    NV_REQUIRE(T < (1LL << 31), NV_ERR_UNSUPPORTED, "nv_moe_route_softmax: launch too large");
+    hipLaunchKernelGGL(moe_route_softmax_kernel, dim3((unsigned)T), dim3(64), 0, (hipStream_t)stream, logits, correction, ids,
+                       weights, E, top, scale);
+    return check_launch("nv_moe_route_softmax");
 }

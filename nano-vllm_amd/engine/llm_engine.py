@@ -85,6 +85,11 @@ class LLMEngine:
         step does; nothing is sampled.  `end`: requests that are finished after this step; their blocks and state
         slot go back.  Returns float32 logits [asked places, vocab] in the order of the entries."""
         plan, rows = [], []
+        max_pos = getattr(self.runner.cfg, "max_position_embeddings", None)
+        for rid, tokens, _ in entries:
+            held = len(self._replayed[rid]) if rid in self._replayed else 0
+            if max_pos is not None and held + len(tokens) > max_pos:
+                raise ValueError(f"{rid}: {held + len(tokens)} tokens exceed max_position_embeddings ({max_pos})")
         for rid, tokens, want in entries:
             seq = self._replayed.get(rid)
             if seq is None:

@@ -21,3 +21,10 @@ class GeluTanhAndMul(nn.Module):
 
     def forward(self, x: torch.Tensor) -> torch.Tensor:
         return ops.gelu_tanh_and_mul(x)
+
+
+class SiluAndMulRows(nn.Module):
+    """silu(gate) * up for x = [gate | up] of any width (the HIP kernel ``nv_silu_and_mul_rows``; bfloat16 or float32)."""
+
+    def forward(self, x: torch.Tensor) -> torch.Tensor:
+        return ops.silu_and_mul_rows(x)

@@ -12,6 +12,11 @@ base^(-2i/R), optionally blended for long contexts: with dim(t) = R ln(original 
 lo = max(floor(dim(fast)), 0), hi = min(ceil(dim(slow)), R - 1) and ramp_i = clamp((i - lo) / max(hi - lo, 0.001), 0, 1)
 the frequency becomes f_i / factor * ramp_i + f_i (1 - ramp_i), and cos and sin are multiplied by 0.1 ln(factor) + 1.
 The module owns no cache (a layer that runs several times per forward has one per run).
+
+``UnrotatedLatentAttention``: the same without positions, so the cached row is the latent alone and serves as key and value;
+a learned sink per head may join the softmax denominator; a layer may read a cache that another layer fills (it then has no
+latent of its own).  ``HeadLinear``: the per-head up-projections around it, as one launch each on [T, heads * size] rows,
+optionally multiplied by a sigmoid gate on the way out.
 """
 from __future__ import annotations
 
@@ -64,3 +69,36 @@ class LatentAttention(nn.Module):
         o = ops.attn_scoremod_paged(q_full, k_cache, v_cache, ctx.cu_seqlens_q, ctx.cu_seqlens_k, ctx.block_tables,
                                     self.scale, 0.0, None, None, ctx.max_seqlen_q, ctx.max_seqlen_k, singles)
         return o.view(q.shape[0], self.num_heads, self.rank)
+
+
+class UnrotatedLatentAttention(nn.Module):
+    def __init__(self, num_heads: int, rank: int, scale: float, eps: float, own_latent: bool = True, use_sink: bool = False,
+                 device=None):
+        super().__init__()
+        self.num_heads, self.rank, self.scale, self.eps = num_heads, rank, float(scale), eps
+        f32 = dict(dtype=torch.float32, device=device)
+        self.latent_norm = nn.Parameter(torch.ones(rank, **f32)) if own_latent else None
+        self.sink = nn.Parameter(torch.zeros(num_heads, **f32)) if use_sink else None
+
+    def forward(self, q_lat: torch.Tensor, c_raw: torch.Tensor | None, k_cache: torch.Tensor, v_cache: torch.Tensor) -> torch.Tensor:
+        """q_lat [T, H * rank]: the queries in latent space; c_raw [T, rank]: the step's latents as projected (None: another
+        layer has stored them); k_cache [num_blocks, block_size, 1, rank], v_cache a view of it.  Returns [T, H * rank]."""
+        ctx = get_context()
+        if self.latent_norm is not None:
+            ops.latent_store(c_raw, self.latent_norm, ctx.slot_mapping, k_cache, self.eps)
+        singles = -1 if ctx.num_decode_seqs is None else int(ctx.num_decode_seqs > 0)
+        return ops.attn_scoremod_paged(q_lat.view(-1, self.num_heads, self.rank), k_cache, v_cache, ctx.cu_seqlens_q,
+                                       ctx.cu_seqlens_k, ctx.block_tables, self.scale, 0.0, self.sink, None, ctx.max_seqlen_q,
+                                       ctx.max_seqlen_k, singles)
+
+
+class HeadLinear(nn.Module):
+    """y[t, h] = weight[h] x[t, h], weight [heads, out, in]."""
+
+    def __init__(self, heads: int, n_in: int, n_out: int, dtype=None, device=None):
+        super().__init__()
+        self.weight = nn.Parameter(torch.zeros(heads, n_out, n_in, dtype=dtype, device=device))
+
+    def forward(self, x: torch.Tensor, gate: torch.Tensor | None = None) -> torch.Tensor:
+        """x [T, heads * in]; gate [T, heads * out] or None: the result times sigmoid(gate).  Returns [T, heads * out]."""
+        return ops.head_linear(x, self.weight, gate)

@@ -11,6 +11,11 @@ unit D (silu(G h) * (U h)), and the caller weights the outputs (each expert coun
 correction, among the experts of the best consecutive blocks of experts (a block's merit: the sum of its top two biased
 scores); the weights are the plain scores of the chosen, used as they are.  ``SquaredReluExperts``: experts
 without a gate, D max(U h, 0)^2, weighted by the router's weights.
+
+``SoftmaxRouter``: scores are a softmax over all experts; the choice is made on score + a per-expert correction; the weights
+are the plain scores of the chosen times a constant.  ``SiluExperts``: D (silu(G h) * (U h)) of the chosen, weighted.  The last
+experts a router scores may be identity experts: they have no tensors, ``SiluExperts`` leaves their rows unwritten, and the
+stream boundary adds their weight times the experts' input instead.
 """
 from __future__ import annotations
 
@@ -62,3 +67,25 @@ class SquaredReluExperts(nn.Module):
         """h [T, W]; ids / weights [T, top]; up [E, ff, W]; down [E, W, ff].  Returns the weighted expert outputs
         [T, top, W] float32."""
         return ops.moe_relu2_experts(h, ids, weights, up, down)
+
+
+class SoftmaxRouter(nn.Module):
+    def __init__(self, experts: int, top: int, scale: float = 1.0, device=None):
+        """experts: all that are scored, identity experts included."""
+        super().__init__()
+        if not 1 <= top <= experts:
+            raise ValueError("top must lie in 1 .. experts")
+        self.experts, self.top, self.scale = int(experts), int(top), float(scale)
+        self.correction = nn.Parameter(torch.zeros(experts, dtype=torch.float32, device=device))
+
+    def forward(self, logits: torch.Tensor) -> tuple:
+        """logits [T, experts] float32 -> (ids [T, top] int32, weights [T, top] float32)."""
+        return ops.moe_route_softmax(logits, self.correction, self.top, self.scale)
+
+
+class SiluExperts(nn.Module):
+    def forward(self, h: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, gate_up: torch.Tensor,
+                down: torch.Tensor) -> torch.Tensor:
+        """h [T, W]; ids / weights [T, top]; gate_up [E, 2 ff, W]; down [E, W, ff].  Returns the weighted expert outputs
+        [T, top, W] float32; rows of ids >= E are not written."""
+        return ops.moe_silu_experts(h, ids, weights, gate_up, down)

@@ -7,6 +7,11 @@ carried in ``prev_state[slot]``.  ``stream_boundary_pair``: everything that happ
 ONE launch: the sublayers' outputs are added (matmul-dtype tensors, fp32 parts such as the outputs of the chosen
 experts times a common weight, and outputs that are RMS-normed on their way in), and up to two norms of the result are
 written side by side in float32 for the next layer's sublayers.  ``ReluSquared``: max(x, 0)^2.
+
+``PositionEmbedding``: a row of a token table plus a row of a learned position table, as the float32 stream.
+``layernorm_pair_boundary``: the boundary of a stream that is read through two LAYER norms with biases: the sublayers'
+outputs and the routed experts' (identity experts add their weight times what the experts read) go in, both norms of the
+result come out in the matmul dtype, the second also in float32 for a router.
 """
 from __future__ import annotations
 
@@ -17,6 +22,7 @@ from .. import ops
 from ..utils.cache_context import get_context
 
 stream_boundary_pair = ops.stream_boundary_pair
+layernorm_pair_boundary = ops.stream_layernorm_pair
 
 
 class HashedBigramEmbedding(nn.Module):
@@ -40,3 +46,14 @@ class HashedBigramEmbedding(nn.Module):
 class ReluSquared(nn.Module):
     def forward(self, x: torch.Tensor) -> torch.Tensor:
         return ops.relu_squared(x)
+
+
+class PositionEmbedding(nn.Module):
+    def __init__(self, vocab: int, max_positions: int, width: int, dtype=None, device=None):
+        super().__init__()
+        self.weight = nn.Parameter(torch.zeros(vocab, width, dtype=dtype, device=device))
+        self.pos = nn.Parameter(torch.zeros(max_positions, width, dtype=dtype, device=device))
+
+    def forward(self, ids: torch.Tensor, positions: torch.Tensor) -> torch.Tensor:
+        """ids, positions [T] int64; returns the stream [T, W] float32."""
+        return ops.embed_positions(ids, positions, self.weight, self.pos)

@@ -119,6 +119,16 @@ def _tutedra_model(cfg, dtype=torch.bfloat16, device="cuda", **kw):
     return TutedraForCausalLM(cfg, dtype=dtype, device=device, **kw)
 
 
+def _nekodra_config(raw: dict):
+    from .nekodra import NekodraConfig
+    return NekodraConfig.from_dict(raw)
+
+
+def _nekodra_model(cfg, dtype=torch.bfloat16, device="cuda", **kw):
+    from .nekodra import NekodraForCausalLM
+    return NekodraForCausalLM(cfg, dtype=dtype, device=device, **kw)
+
+
 register(["Qwen3ForCausalLM", "Qwen3"], _qwen3_config, lambda cfg, **kw: _qwen3_model(cfg, **kw))
 register(["LlamaForCausalLM", "Llama"], lambda raw: _qwen3_config({**raw, "qk_norm": False}),
          lambda cfg, **kw: _qwen3_model(cfg, **kw))
@@ -126,3 +136,4 @@ register(["Buvalix", "BuvalixForCausalLM"], _buvalix_config, _buvalix_model)
 register(["Benarax", "BenaraxForCausalLM"], _benarax_config, _benarax_model)
 register(["Divadra", "DivadraForCausalLM"], _divadra_config, _divadra_model)
 register(["Tutedra", "TutedraForCausalLM"], _tutedra_config, _tutedra_model)
+register(["Nekodra", "NekodraForCausalLM"], _nekodra_config, _nekodra_model)

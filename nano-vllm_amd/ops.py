@@ -1098,10 +1098,11 @@ def attn_chunk_sigmoid_paged(q: torch.Tensor, k_cache: torch.Tensor, v_cache: to
     return out
 
 
-def moe_table_experts(h: torch.Tensor, ids: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor) -> torch.Tensor:
-    """Experts chosen by a table: h [T, W]; ids [T, top] int32 (the experts of every token, distinct per row); gate_up
-    [E, 2 ff, W]; down [E, W, ff].  Expert: D (silu(G h) * (U h)).  Returns the UNWEIGHTED outputs of every token's
-    experts, [T, top, W] float32 (the stream update scales and sums them)."""
+def moe_silu_experts(h: torch.Tensor, ids: torch.Tensor, weights: Optional[torch.Tensor], gate_up: torch.Tensor,
+                     down: torch.Tensor) -> torch.Tensor:
+    """Chosen experts D (silu(G h) * (U h)): h [T, W]; ids [T, top] int32 (distinct per row); weights [T, top] float32, or None
+    for 1; gate_up [E, 2 ff, W]; down [E, W, ff].  Returns the weighted outputs [T, top, W] float32 (the stream update sums
+    them).  The rows of choices whose id is not below E are NOT written."""
     dt = _dt(h, "h")
     _rows2d(h, "h")
     T, W = h.shape
@@ -1117,7 +1118,9 @@ def moe_table_experts(h: torch.Tensor, ids: torch.Tensor, gate_up: torch.Tensor,
     out = torch.empty((T, top, W), dtype=torch.float32, device=dev)
     if T == 0:
         return out
-    wgt = torch.ones((T, top), dtype=torch.float32, device=dev)
+    if weights is None:
+        weights = torch.ones((T, top), dtype=torch.float32, device=dev)
+    _need(weights.shape == (T, top), "weights must be [T, top]")
     rows = dll.nv_moe_tile_rows(P, E)
     tiles = dll.nv_moe_max_tiles(P, E, rows)
     sorted_pairs = torch.empty(P, dtype=torch.int32, device=dev)
@@ -1127,9 +1130,14 @@ def moe_table_experts(h: torch.Tensor, ids: torch.Tensor, gate_up: torch.Tensor,
     _lib.check(dll.nv_moe_gate_up_act(h.data_ptr(), h.stride(0), gate_up.data_ptr(), sorted_pairs.data_ptr(),
                                       meta.data_ptr(), y.data_ptr(), dt, P, E, int(top), W, ff, float("inf"), 1.0, 0.0,
                                       rows, s), "nv_moe_gate_up_act", dll)
-    _lib.check(dll.nv_moe_down(y.data_ptr(), down.data_ptr(), sorted_pairs.data_ptr(), meta.data_ptr(), wgt.data_ptr(),
+    _lib.check(dll.nv_moe_down(y.data_ptr(), down.data_ptr(), sorted_pairs.data_ptr(), meta.data_ptr(), _f32c(weights, "weights"),
                                out.data_ptr(), dt, P, E, W, ff, rows, s), "nv_moe_down", dll)
     return out
+
+
+def moe_table_experts(h: torch.Tensor, ids: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor) -> torch.Tensor:
+    """Experts chosen by a table, unweighted (the stream update scales and sums them): moe_silu_experts with weight 1."""
+    return moe_silu_experts(h, ids, None, gate_up, down)
 
 
 # ---------------------------------------------------------------------------------------------------------
@@ -1362,3 +1370,139 @@ def moe_relu2_experts(h: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor,
     _lib.check(dll.nv_moe_down(y.data_ptr(), down.data_ptr(), sorted_pairs.data_ptr(), meta.data_ptr(), weights.data_ptr(),
                                out.data_ptr(), dt, P, E, W, ff, rows, s), "nv_moe_down", dll)
     return out
+
+
+# ---------------------------------------------------------------------------------------------------------
+# fp32 stream read through two layer norms with biases, learned positions, latents without a rotated part, per-head
+# products, softmax routing with a selection correction and experts that hand their input through.
+# ---------------------------------------------------------------------------------------------------------
+def embed_positions(ids: torch.Tensor, positions: torch.Tensor, embed: torch.Tensor, pos: torch.Tensor) -> torch.Tensor:
+    """embed[ids] + pos[positions] as a float32 stream [T, W]."""
+    dt = _dt(embed, "embed")
+    T = ids.numel()
+    for t, n in ((ids, "ids"), (positions, "positions")):
+        _need(t.is_cuda and t.dtype == torch.int64 and t.is_contiguous() and t.numel() == T,
+              f"{n} must be a contiguous int64 [tokens] GPU tensor")
+    _need(embed.dim() == 2 and pos.dim() == 2 and embed.is_contiguous() and pos.is_contiguous() and pos.is_cuda
+          and pos.dtype == embed.dtype and pos.shape[1] == embed.shape[1], "embed and pos must be contiguous tables of one width and dtype")
+    x = torch.empty((T, embed.shape[1]), dtype=torch.float32, device=embed.device)
+    dll = _lib.mixers()
+    rc = dll.nv_embed_positions(ids.data_ptr(), positions.data_ptr(), embed.data_ptr(), pos.data_ptr(), x.data_ptr(), dt, T,
+                                embed.shape[1], embed.shape[0], pos.shape[0], _stream(embed))
+    _lib.check(rc, "nv_embed_positions", dll)
+    return x
+
+
+def stream_layernorm_pair(x: torch.Tensor, adds=(), routed: Optional[tuple] = None, norm_a: Optional[tuple] = None,
+                          norm_b: Optional[tuple] = None, eps: float = 1e-5, out_dtype: Optional[torch.dtype] = None,
+                          want_f32_b: bool = False):
+    """One layer boundary of an fp32 stream x [T, W], in place: x += sum(adds) + the routed experts' outputs.
+    routed = (parts [T, n, W] float32 already weighted, ids [T, n] int32, weights [T, n] float32, experts, through [T, W]):
+    choices with ids >= experts add their weight times `through`, and their parts are not read; ids None: every part
+    counts.  norm_a / norm_b: (weight, bias) of up to two layer norms of the updated stream.  Returns (a, b, b32): the norms
+    in out_dtype, the second also in float32 if want_f32_b; None for what was not asked for."""
+    _need(x.is_cuda and x.dtype == torch.float32 and x.dim() == 2 and x.is_contiguous(),
+          "the stream must be a contiguous float32 [tokens, width] GPU tensor")
+    rows, cols = x.shape
+    adds = list(adds)
+    _need(len(adds) <= 2, "at most two added tensors")
+    parts = ids = weights = through = None
+    experts = n_parts = 0
+    if routed is not None:
+        parts, ids, weights, experts, through = routed
+        n_parts = parts.shape[1]
+        _need(parts.is_cuda and parts.dtype == torch.float32 and parts.is_contiguous() and parts.shape == (rows, n_parts, cols),
+              "parts must be contiguous float32 [T, n, W]")
+        if ids is not None:
+            _need(ids.is_cuda and ids.dtype == torch.int32 and ids.is_contiguous() and ids.shape == (rows, n_parts)
+                  and weights is not None and weights.shape == ids.shape, "ids (int32) and weights (float32) must be [T, n]")
+        else:
+            weights = through = None
+    ins = adds + ([through] if through is not None else [])
+    dt_t = out_dtype or (ins[0].dtype if ins else torch.float32)
+    _need(dt_t in (_BF16, torch.float32), "the matmul dtype must be bfloat16 or float32")
+    for t in ins:
+        _rows2d(t, "input")
+        _need(t.shape == x.shape and t.dtype == dt_t and t.is_cuda, "inputs must match the stream's shape, in the matmul dtype")
+    for pair in (norm_a, norm_b):
+        if pair is not None:
+            _need(pair[0].numel() == cols and pair[1].numel() == cols, "norm weights and biases must be [width]")
+    new = lambda dtype: torch.empty((rows, cols), dtype=dtype, device=x.device)
+    a = new(dt_t) if norm_a is not None else None
+    b = new(dt_t) if norm_b is not None else None
+    b32 = new(torch.float32) if norm_b is not None and want_f32_b else None
+    st = lambda t: t.stride(0) if t is not None else 0
+    a1, a2 = (adds + [None, None])[:2]
+    fp = lambda t, n: _f32c(t, n) or None
+    dll = _lib.mixers()
+    rc = dll.nv_stream_layernorm_pair(
+        x.data_ptr(), _ptr(a1), st(a1), _ptr(a2), st(a2), _ptr(parts), _ptr(ids), fp(weights, "weights"), n_parts, int(experts),
+        _ptr(through), st(through), fp(norm_a[0] if norm_a else None, "weight"), fp(norm_a[1] if norm_a else None, "bias"),
+        fp(norm_b[0] if norm_b else None, "weight"), fp(norm_b[1] if norm_b else None, "bias"), float(eps), _ptr(a), _ptr(b),
+        _ptr(b32), _lib.DTYPE_BF16 if dt_t == _BF16 else _lib.DTYPE_F32, rows, cols, _stream(x))
+    _lib.check(rc, "nv_stream_layernorm_pair", dll)
+    return a, b, b32
+
+
+def silu_and_mul_rows(x: torch.Tensor) -> torch.Tensor:
+    """y = silu(gate) * up for x = [gate | up] along the last dimension, any width (fp32 arithmetic, one rounding)."""
+    _rows2d(x, "x")
+    dt = _dt(x, "x")
+    inter = x.shape[1] // 2
+    y = torch.empty((x.shape[0], inter), dtype=x.dtype, device=x.device)
+    dll = _lib.mixers()
+    rc = dll.nv_silu_and_mul_rows(x.data_ptr(), x.stride(0), y.data_ptr(), dt, x.shape[0], inter, _stream(x))
+    _lib.check(rc, "nv_silu_and_mul_rows", dll)
+    return y
+
+
+def latent_store(ckv: torch.Tensor, latent_weight: torch.Tensor, slot_mapping: torch.Tensor, cache: torch.Tensor, eps: float) -> None:
+    """cache[slot] = ckv / rms(ckv) * latent_weight per token; ckv [T, rank]; cache [num_blocks, block_size, 1, rank]."""
+    _rows2d(ckv, "ckv")
+    dt = _dt(ckv, "ckv")
+    T, rank = ckv.shape
+    _i32(slot_mapping, "slot_mapping")
+    _need(slot_mapping.numel() == T, "slot_mapping length != number of tokens")
+    _need(latent_weight.numel() == rank, "latent weight must be [rank]")
+    _need(cache.is_cuda and cache.is_contiguous() and cache.dtype == ckv.dtype and cache.shape[2:] == (1, rank),
+          "the cache must be contiguous [num_blocks, block_size, 1, rank] of ckv's dtype")
+    dll = _lib.mixers()
+    rc = dll.nv_latent_store(ckv.data_ptr(), ckv.stride(0), _f32c(latent_weight, "latent_weight"), slot_mapping.data_ptr(),
+                             cache.data_ptr(), cache.shape[0] * cache.shape[1], dt, T, rank, float(eps), _stream(ckv))
+    _lib.check(rc, "nv_latent_store", dll)
+
+
+def head_linear(x: torch.Tensor, w: torch.Tensor, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Per-head product y[t, h] = w[h] x[t, h]: x [T, H * K] (row stride free), w [H, N, K]; with `gate` [T, H * N] the result
+    is multiplied by sigmoid(gate).  Returns [T, H * N]."""
+    _rows2d(x, "x")
+    dt = _dt(x, "x")
+    T = x.shape[0]
+    _need(w.is_cuda and w.dtype == x.dtype and w.is_contiguous() and w.dim() == 3, "w must be contiguous [H, N, K] of x's dtype")
+    H, N, K = w.shape
+    _need(x.shape[1] == H * K, "x must be [T, H * K]")
+    if gate is not None:
+        _rows2d(gate, "gate")
+        _need(gate.is_cuda and gate.dtype == x.dtype and gate.shape == (T, H * N), "gate must be [T, H * N] of x's dtype")
+    y = torch.empty((T, H * N), dtype=x.dtype, device=x.device)
+    dll = _lib.mixers()
+    rc = dll.nv_head_linear(x.data_ptr(), x.stride(0), w.data_ptr(), _ptr(gate), gate.stride(0) if gate is not None else 0,
+                            y.data_ptr(), dt, T, H, N, K, _stream(x))
+    _lib.check(rc, "nv_head_linear", dll)
+    return y
+
+
+def moe_route_softmax(logits: torch.Tensor, correction: Optional[torch.Tensor], top: int, scale: float) -> tuple:
+    """Softmax scores over all experts, choice on score + correction, weights = scale * score of the chosen: logits [T, E]
+    float32 -> (ids [T, top] int32, weights [T, top] float32)."""
+    _need(logits.is_cuda and logits.dtype == torch.float32 and logits.is_contiguous() and logits.dim() == 2,
+          "logits must be contiguous float32 [T, E]")
+    T, E = logits.shape
+    _need(correction is None or correction.numel() == E, "correction must be [E]")
+    ids = torch.empty((T, top), dtype=torch.int32, device=logits.device)
+    wgt = torch.empty((T, top), dtype=torch.float32, device=logits.device)
+    dll = _lib.mixers()
+    rc = dll.nv_moe_route_softmax(logits.data_ptr(), _f32c(correction, "correction") or None, ids.data_ptr(), wgt.data_ptr(), T, E,
+                                  int(top), float(scale), _stream(logits))
+    _lib.check(rc, "nv_moe_route_softmax", dll)
+    return ids, wgt
