@@ -74,6 +74,9 @@ def parse():
     ap.add_argument("--tutedra", action="store_true",
                     help="instead of the default workload: the Tutedra kernels and model beside Benarax at equal sizes "
                          "(one GPU, random weights), one JSON line")
+    ap.add_argument("--nekodra", action="store_true",
+                    help="instead of the default workload: the Nekodra kernels and model beside Benarax at equal sizes "
+                         "(one GPU, random weights), one JSON line")
     return ap.parse_args()
 
 
@@ -811,6 +814,12 @@ def main():
             raise SystemExit("bench.py needs a GPU (the hot path has no CPU implementation)")
         from tools.tutedra_bench import run as tutedra_run
         print(json.dumps(tutedra_run("cuda:0")))
+        return
+    if args.nekodra:
+        if not torch.cuda.is_available():
+            raise SystemExit("bench.py needs a GPU (the hot path has no CPU implementation)")
+        from tools.nekodra_bench import run as nekodra_run
+        print(json.dumps(nekodra_run("cuda:0")))
         return
     if args.divadra:
         if not torch.cuda.is_available():
