@@ -1,0 +1,75 @@
+"""Nekodra with configurations drawn at random (sizes, head counts, which layers share latents, score scales, experts,
+identity experts, top, router scale, shared experts), through the engine against the plain oracle: what holds for the
+hand-made configurations of the other tests must hold for any, in particular sizes that are no multiple of a vector or of a
+matrix tile, and values that hand-made configurations happen to make equal or 1.  CPU: eager stand-ins; gpu: the HIP kernels
+in float32 (tight) and bfloat16 (rounding-sized)."""
+import math
+import os
+import random
+
+import pytest
+import torch
+
+from nekodra_util import make_engine, oracle_logits, per_position, random_checkpoint, replay
+
+BACKENDS = [pytest.param(("cpu", torch.float32), id="cpu-f32"),
+            pytest.param(("cuda", torch.float32), id="gpu-f32", marks=pytest.mark.gpu),
+            pytest.param(("cuda", torch.bfloat16), id="gpu-bf16", marks=pytest.mark.gpu)]
+
+
+def draw_config(seed: int) -> dict:
+    rng = random.Random(seed)
+    layers = []
+    for i in range(rng.randint(1, 6)):
+        dim = rng.choice([4, 7, 8, 16, 24, 32, 40, 64])
+        mixer = {"heads": rng.randint(1, 9), "dim": dim, "vdim": rng.choice([3, 8, 16, 20, 32, 56, 64]),
+                 "kv_rank": rng.choice([4, 9, 16, 32, 36, 48, 64, 80, 96, 112, 128, 192]), "scale": rng.choice([0.5, 1.0, 1.5]) / math.sqrt(dim)}
+        own = [j for j, L in enumerate(layers) if "kv_from" not in L["mixer"]]
+        if own and rng.random() < 0.5:
+            mixer["kv_from"] = rng.choice(own)
+            mixer["kv_rank"] = layers[mixer["kv_from"]]["mixer"]["kv_rank"]
+        mlp = None
+        if rng.random() < 0.85:
+            experts, identity = rng.randint(1, 12), rng.randint(0, 4)
+            mlp = {"kind": "moe", "expert": {"ff": rng.choice([4, 8, 12, 20, 33, 72])},
+                   "router": {"experts": experts, "identity": identity, "top": rng.randint(1, min(experts + identity, 6)),
+                              "scale": rng.choice([1.0, 0.7, 3.0])}}
+            if rng.random() < 0.6:
+                mlp["shared"] = {"ff": rng.choice([3, 8, 16, 40])}
+        layers.append({"type": "latent_attention", "mixer": mixer, "mlp": mlp})
+    return {"architecture": "Nekodra", "layers": layers, "norm": {"eps": rng.choice([1e-6, 1e-5, 1e-3])}, "vocab": rng.randint(20, 120),
+            "width": rng.choice([8, 12, 20, 37, 64, 72, 128]), "max_positions": rng.choice([40, 64, 1000])}
+
+
+@pytest.fixture(params=BACKENDS)
+def backend(request):
+    return request.param
+
+
+@pytest.mark.parametrize("seed", range(int(os.environ.get("NV_RANDOM_CONFIGS", "14"))))      # more for a longer sweep
+def test_random_configuration(seed, backend):
+    dev, dtype = backend
+    cfg = draw_config(seed)
+    ck = random_checkpoint(cfg, seed=100 + seed, correction=seed % 5 != 1)
+    g = torch.Generator().manual_seed(seed)
+    V = cfg["vocab"]
+    p = {"a": torch.randint(0, V, (29,), generator=g).tolist(), "b": torch.randint(0, V, (7,), generator=g).tolist(),
+         "c": torch.randint(0, V, (40,), generator=g).tolist()}
+    portions = {"a": [6, 1, 1, 14, 2, 1], "b": [1], "c": [2, 3, 30, 1]}
+    got = replay(make_engine(cfg, ck, dev, dtype, block_size=4, num_blocks=40, max_seqs=3), p, portions, order={"b": 2, "c": 1})
+    # Per position, against what the oracle's own bfloat16 evaluation loses there.  float32: every position within 1e-4, or
+    # within 2 % of that loss where it is large.  bfloat16: a fault moves most positions, rounding (two experts with almost
+    # equal scores) moves a few by more than three times the oracle's loss.
+    errs, noises = [], []
+    for i in p:
+        want = oracle_logits(cfg, ck, p[i])
+        errs.append(per_position(got[i], want))
+        noises.append(per_position(oracle_logits(cfg, ck, p[i], torch.bfloat16), want))
+    err, noise = torch.cat(errs), torch.cat(noises)
+    if dtype == torch.float32:
+        assert bool((err < torch.clamp(0.02 * noise, min=1e-4)).all()), (seed, dev, err.max().item())
+    else:
+        limit = 3 * torch.clamp(noise, min=noise.median().item()) + 1e-3
+        over = int((err > limit).sum())
+        assert over <= max(1, err.numel() // 10), (seed, (err / limit).topk(5).values.tolist())
+        assert err.median().item() <= 2 * noise.median().item() + 1e-3, (seed, err.median().item(), noise.median().item())
