@@ -438,6 +438,23 @@ NV_API int nv_latent_store(const void* ckv, int64_t ckv_stride, const float* lat
 NV_API int nv_head_linear(const void* x, int64_t x_stride, const void* w, const void* gate, int64_t gate_stride, void* y,
                           int dtype, int64_t T, int H, int N, int K, void* stream);
 
+/*
+ * Causal paged attention in latent space on the matrix cores (bf16): all H query heads of a token attend to one cached row of
+ * D columns per key, whose first Dv columns are the value; fp32 scores times `scale` (> 0) and softmax, exp(sink[h]) joins
+ * the denominator if sink.  q: [T, H, D], cache: [num_blocks, block_size, D], out: [T, H, Dv], all contiguous and 16-byte
+ * aligned.  Lengths and tables as for nv_attn_scoremod_paged, but max_seqlen_q / max_seqlen_k must be given.
+ * nv_attn_latent_ok: whether a kernel is built for the sizes (rows and values in certain multiples of 32, blocks of a
+ * multiple of 64 tokens); nv_attn_scoremod_paged_vld takes the rest.
+ */
+NV_API int nv_attn_latent_ok(int D, int Dv, int block_size);
+NV_API int64_t nv_attn_latent_workspace_bytes(int num_seqs, int64_t T, int H, int D, int Dv, int max_seqlen_q,
+                                              int max_seqlen_k);
+NV_API int nv_attn_latent_paged(const void* q, const void* cache, void* out, const int32_t* cu_seqlens_q,
+                                const int32_t* cu_seqlens_k, const int32_t* block_tables, int num_seqs,
+                                int max_blocks_per_seq, int64_t T, int H, int D, int Dv, int64_t num_blocks, int block_size,
+                                float scale, const float* sink, int max_seqlen_q, int max_seqlen_k, int single_rows,
+                                void* workspace, int64_t workspace_bytes, void* stream);
+
 #ifdef __cplusplus
 }
 #endif

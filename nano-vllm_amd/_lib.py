@@ -135,6 +135,10 @@ MIXERS_PROTOTYPES = {
     "nv_silu_and_mul_rows": (_i32, [_vp, _i64, _vp, _i32, _i64, _i32, _vp]),
     "nv_latent_store": (_i32, [_vp, _i64, _vp, _vp, _vp, _i64, _i32, _i64, _i32, _f32, _vp]),
     "nv_head_linear": (_i32, [_vp, _i64, _vp, _vp, _i64, _vp, _i32, _i64, _i32, _i32, _i32, _vp]),
+    "nv_attn_latent_ok": (_i32, [_i32, _i32, _i32]),
+    "nv_attn_latent_workspace_bytes": (_i64, [_i32, _i64, _i32, _i32, _i32, _i32, _i32]),
+    "nv_attn_latent_paged": (_i32, [_vp, _vp, _vp, _vp, _vp, _vp, _i32, _i32, _i64, _i32, _i32, _i32, _i64, _i32, _f32, _vp, _i32,
+                                    _i32, _i32, _vp, _i64, _vp]),
     "nv_moe_up_relu2": (_i32, [_vp, _i64, _vp, _vp, _vp, _vp, _i32, _i64, _i32, _i32, _i32, _i32, _i32, _vp]),
 }
 DTYPE_BF16, DTYPE_F32 = 0, 1

@@ -5,7 +5,8 @@ all heads share.  With the key up-projection moved to the query (q_lat = Uk_h^T 
 value up-projection moved behind the attention, this is multi-query attention with key [c | k_r] and value c:
 
   * ``nv_latent_prep_store``    normalises c, rotates k_r and the queries' rotated part, scatters the cache rows,
-  * ``nv_attn_scoremod_paged``  the framework's paged attention with free head sizes (one kv head, fp32 softmax).
+  * ``nv_attn_latent_paged``    attention on the matrix cores over rows that serve as key and value (bfloat16, built row
+                                sizes), or ``nv_attn_scoremod_paged``, the general launch with free head sizes.
 
 Rotary: pair i is turned by position * freq[i]; the pairing is (2i, 2i+1) or (i, i + R/2).  The frequencies are
 base^(-2i/R), optionally blended for long contexts: with dim(t) = R ln(original / (2 pi t)) / (2 ln base),
@@ -66,8 +67,8 @@ class LatentAttention(nn.Module):
         q_full = ops.latent_prep_store(q, q_lat, ckv, self.latent_norm, self.freq, self.mag, self.interleaved, positions,
                                        ctx.slot_mapping, k_cache, v_cache, self.rot_dim, self.eps)
         singles = -1 if ctx.num_decode_seqs is None else int(ctx.num_decode_seqs > 0)
-        o = ops.attn_scoremod_paged(q_full, k_cache, v_cache, ctx.cu_seqlens_q, ctx.cu_seqlens_k, ctx.block_tables,
-                                    self.scale, 0.0, None, None, ctx.max_seqlen_q, ctx.max_seqlen_k, singles)
+        o = ops.attn_latent_paged(q_full, k_cache, v_cache, ctx.cu_seqlens_q, ctx.cu_seqlens_k, ctx.block_tables,
+                                  self.scale, None, ctx.max_seqlen_q, ctx.max_seqlen_k, singles)
         return o.view(q.shape[0], self.num_heads, self.rank)
 
 
@@ -87,9 +88,9 @@ class UnrotatedLatentAttention(nn.Module):
         if self.latent_norm is not None:
             ops.latent_store(c_raw, self.latent_norm, ctx.slot_mapping, k_cache, self.eps)
         singles = -1 if ctx.num_decode_seqs is None else int(ctx.num_decode_seqs > 0)
-        return ops.attn_scoremod_paged(q_lat.view(-1, self.num_heads, self.rank), k_cache, v_cache, ctx.cu_seqlens_q,
-                                       ctx.cu_seqlens_k, ctx.block_tables, self.scale, 0.0, self.sink, None, ctx.max_seqlen_q,
-                                       ctx.max_seqlen_k, singles)
+        return ops.attn_latent_paged(q_lat.view(-1, self.num_heads, self.rank), k_cache, v_cache, ctx.cu_seqlens_q,
+                                     ctx.cu_seqlens_k, ctx.block_tables, self.scale, self.sink, ctx.max_seqlen_q,
+                                     ctx.max_seqlen_k, singles)
 
 
 class HeadLinear(nn.Module):

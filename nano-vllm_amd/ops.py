@@ -1492,6 +1492,41 @@ def head_linear(x: torch.Tensor, w: torch.Tensor, gate: Optional[torch.Tensor] =
     return y
 
 
+def attn_latent_paged(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, cu_seqlens_q: torch.Tensor,
+                      cu_seqlens_k: torch.Tensor, block_tables: torch.Tensor, scale: float, sink: Optional[torch.Tensor] = None,
+                      max_seqlen_q: int = 0, max_seqlen_k: int = 0, single_rows: int = -1) -> torch.Tensor:
+    """Causal paged attention of q [T, H, D] over ONE cached row per token, k_cache [num_blocks, block_size, 1, D], whose first
+    columns are the value (v_cache a column range of it, or a cache of its own); returns [T, H * Dv].  bfloat16 rows of the
+    built sizes take the matrix-core kernels, everything else the general attention launch."""
+    dll = _lib.mixers()
+    T, H, D = q.shape
+    nb, bs, G, _ = k_cache.shape
+    Dv = v_cache.shape[3]
+    if not (q.dtype == _BF16 and G == 1 and v_cache.data_ptr() == k_cache.data_ptr() and q.is_contiguous() and scale > 0
+            and max_seqlen_q > 0 and max_seqlen_k > 0 and dll.nv_attn_latent_ok(D, Dv, bs)):
+        return attn_scoremod_paged(q, k_cache, v_cache, cu_seqlens_q, cu_seqlens_k, block_tables, scale, 0.0, sink, None,
+                                   max_seqlen_q, max_seqlen_k, single_rows)
+    _need(q.is_cuda and k_cache.is_cuda and k_cache.is_contiguous() and k_cache.dtype == q.dtype and k_cache.shape[3] == D
+          and v_cache.stride() == k_cache.stride(), "the cache must be contiguous [num_blocks, block_size, 1, D] of q's dtype")
+    _i32(cu_seqlens_q, "cu_seqlens_q")
+    _i32(cu_seqlens_k, "cu_seqlens_k")
+    B = cu_seqlens_k.numel() - 1
+    _need(cu_seqlens_q.numel() == B + 1, "cu_seqlens_q / cu_seqlens_k length mismatch")
+    _need(block_tables.is_cuda and block_tables.dtype == torch.int32 and block_tables.dim() == 2
+          and block_tables.is_contiguous() and block_tables.shape[0] == B and block_tables.shape[1] * bs >= max_seqlen_k,
+          "block_tables must be a contiguous [B, max_blocks] int32 GPU tensor that covers the longest sequence")
+    _need(sink is None or sink.numel() == H, "sink must be [H]")
+    out = torch.empty((T, H * Dv), dtype=q.dtype, device=q.device)
+    need = dll.nv_attn_latent_workspace_bytes(B, T, H, D, Dv, int(max_seqlen_q), int(max_seqlen_k))
+    ws = _workspace(q.device, need) if need else None
+    rc = dll.nv_attn_latent_paged(q.data_ptr(), k_cache.data_ptr(), out.data_ptr(), cu_seqlens_q.data_ptr(), cu_seqlens_k.data_ptr(),
+                                  block_tables.data_ptr(), B, block_tables.shape[1], T, H, D, Dv, nb, bs, float(scale),
+                                  _f32c(sink, "sink") or None, int(max_seqlen_q), int(max_seqlen_k), int(single_rows), _ptr(ws),
+                                  ws.numel() if ws is not None else 0, _stream(q))
+    _lib.check(rc, "nv_attn_latent_paged", dll)
+    return out
+
+
 def moe_route_softmax(logits: torch.Tensor, correction: Optional[torch.Tensor], top: int, scale: float) -> tuple:
     """Softmax scores over all experts, choice on score + correction, weights = scale * score of the chosen: logits [T, E]
     float32 -> (ids [T, top] int32, weights [T, top] float32)."""

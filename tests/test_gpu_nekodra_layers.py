@@ -155,3 +155,85 @@ def test_silu_experts_leave_identity_choices_alone(dt, T, W, E, extra, top, ff):
     ya, yb = a(h, ids, w, gu, down), b(h, ids, w, gu, down)
     use = ids < E
     assert not use.any() or rel(ya[use], yb[use]) < tol(dt)
+
+
+def reference_rows(q, cache, ctx, scale, sink, Dv):
+    """fp32 attention of q [T, H, D] over the cached rows, sequence by sequence, heads together."""
+    cu_q, cu_k, bs = ctx.cu_seqlens_q.tolist(), ctx.cu_seqlens_k.tolist(), cache.shape[1]
+    out = torch.zeros(q.shape[0], q.shape[1], Dv, device=q.device)
+    for b in range(len(cu_q) - 1):
+        nq, nk = cu_q[b + 1] - cu_q[b], cu_k[b + 1] - cu_k[b]
+        pos = torch.arange(nk, device=q.device)
+        rows = cache.view(-1, q.shape[2])[ctx.block_tables[b].long()[pos // bs] * bs + pos % bs].float()
+        s = torch.matmul(q[cu_q[b]:cu_q[b + 1]].float(), rows.t()) * scale                      # [nq, H, nk]
+        s = s.masked_fill((pos[None, :] > (nk - nq + torch.arange(nq, device=q.device))[:, None])[:, None], float("-inf"))
+        if sink is not None:
+            s = torch.cat([s, sink.view(1, -1, 1).expand(nq, -1, 1)], dim=-1)
+        out[cu_q[b]:cu_q[b + 1]] = torch.matmul(torch.softmax(s, dim=-1)[..., :nk], rows[:, :Dv])
+    return out.reshape(q.shape[0], -1)
+
+
+BUILT = [(32, 32), (64, 64), (96, 96), (128, 128), (160, 160), (192, 192), (224, 224), (256, 256), (320, 320), (384, 384), (512, 512), (160, 128),
+         (192, 128), (256, 192), (320, 256), (576, 512)]
+STEPS = {"mixed": ([5, 1, 200, 2, 1, 77], [5, 140, 333, 66, 1, 640]), "decode": ([1] * 5, [1, 32, 33, 700, 64]), "long_decode": ([1, 1], [5000, 2049]),
+         "long_chunk": ([40], [3000]), "prompts": ([64, 63, 129], [64, 63, 129])}
+
+
+@pytest.mark.parametrize("D,Dv", BUILT, ids=lambda n: str(n))
+@pytest.mark.parametrize("step", sorted(STEPS))
+def test_matrix_core_latent_attention(D, Dv, step):
+    from nanovllm_amd import _lib, ops
+    assert _lib.mixers().nv_attn_latent_ok(D, Dv, 64) == 1
+    n_q, n_k = STEPS[step]
+    for H, bs, sinks in ((16, 64, True), (3, 128, False)) if step != "mixed" else ((33, 64, True), (1, 192, True)):
+        ctx, _ = paged_context(n_q, n_k, bs, sum(-(-n // bs) for n in n_k) + 3, D, DEV)
+        g = torch.Generator().manual_seed(D + H)
+        q = rn(g, sum(n_q), H, D, std=3.0 / D ** 0.5).to(torch.bfloat16)
+        cache = rn(g, sum(-(-n // bs) for n in n_k) + 3, bs, 1, D).to(torch.bfloat16)
+        sink = torch.linspace(-3.0, 6.0, H, device=DEV) if sinks else None
+        got = ops.attn_latent_paged(q, cache, cache[..., :Dv], ctx.cu_seqlens_q, ctx.cu_seqlens_k, ctx.block_tables, 0.9, sink,
+                                    max(n_q), max(n_k), -1)
+        want = reference_rows(q, cache, ctx, 0.9, sink, Dv)
+        assert torch.isfinite(got).all()
+        err = (got.float() - want).view(sum(n_q), -1).norm(dim=-1) / want.norm(dim=-1)
+        assert err.max().item() < 1.2e-2, (H, bs, int(err.argmax()), err.max().item())
+
+
+@pytest.mark.parametrize("D", [64, 160, 512])
+def test_matrix_core_latent_attention_finds_each_key(D):
+    """Every query row is aimed at one key (the score stands 20 above the others): the key at the row's own position, ahead of
+    it (which must weigh nothing), at tile and page edges, and where the launch cuts the keys into ranges."""
+    from nanovllm_amd import ops
+    n_q, n_k, H, bs = [200, 1, 1, 1], [1500, 1500, 4097, 65], 4, 64
+    ctx, _ = paged_context(n_q, n_k, bs, 130, D, DEV)
+    g = torch.Generator().manual_seed(D)
+    T = sum(n_q)
+    unit = torch.nn.functional.normalize(torch.randn(130 * bs, D, generator=g), dim=-1)
+    cache = (unit * D ** 0.5).to(torch.bfloat16).view(130, bs, 1, D).to(DEV)
+    targets, q = [], torch.zeros(T, H, D)
+    cu_q = [0] + torch.tensor(n_q).cumsum(0).tolist()
+    tables = ctx.block_tables.cpu()
+    flat = cache.view(-1, D).float().cpu()
+    for b in range(4):
+        for i in range(n_q[b]):
+            pos = n_k[b] - n_q[b] + i
+            for h in range(H):
+                edges = [pos, 0, 31, 32, 63, 64, 255, 256, 511, 512, 1023, 1024, pos - 1, pos + 1]
+                t = edges[(i * H + h) % len(edges)]
+                t = t if 0 <= t < n_k[b] else pos
+                targets.append((b, t, pos))
+                q[cu_q[b] + i, h] = flat[int(tables[b][t // bs]) * bs + t % bs] * (20.0 / D)
+    got = ops.attn_latent_paged(q.to(torch.bfloat16).to(DEV), cache, cache[..., :D], ctx.cu_seqlens_q, ctx.cu_seqlens_k, ctx.block_tables, 1.0,
+                                None, max(n_q), max(n_k), -1)
+    want = reference_rows(q.to(torch.bfloat16).to(DEV), cache, ctx, 1.0, None, D)
+    rows_got, rows_want = got.float().view(T * H, D), want.view(T * H, D)
+    err = (rows_got - rows_want).norm(dim=-1) / rows_want.norm(dim=-1)
+    seen = torch.tensor([t <= pos for _, t, pos in targets])
+    assert err[seen.to(DEV)].max().item() < 1.2e-2, err.max().item()
+    assert (rows_got - rows_want)[~seen.to(DEV)].abs().max().item() < 0.1
+    for k, (b, t, pos) in enumerate(targets):
+        own = flat[int(tables[b][t // bs]) * bs + t % bs]
+        if t <= pos:
+            assert torch.nn.functional.cosine_similarity(rows_got[k].cpu(), own, dim=0).item() > 0.9, (b, t, pos)
+        else:
+            assert (rows_got[k].cpu() - own).norm() > 0.3 * own.norm(), (b, t, pos)

@@ -65,7 +65,7 @@ def kernel_records(dev):
         out[name] = rec
 
     H = 16
-    for rank, (lr, lR, dim, vdim) in ((160, (128, 32, 128, 96)), (256, (192, 64, 192, 128))):
+    for rank, (lr, lR, dim, vdim) in ((160, (128, 32, 128, 96)), (256, (192, 64, 192, 128)), (512, (512, 64, 128, 128))):
         cases = {"prefill_4x2048": ([2048] * 4, [2048] * 4), "chunk_512_over_8192": ([512], [8192]),
                  "decode_256_seqs_ctx_513_768": ([1] * 256, torch.randint(513, 769, (256,), generator=torch.Generator().manual_seed(1)).tolist()),
                  "decode_32_seqs_ctx_1088": ([1] * 32, [1088] * 32), "decode_8_seqs_ctx_8192": ([1] * 8, [8192] * 8)}
@@ -100,13 +100,15 @@ def kernel_records(dev):
                  dict(nbytes=T * H * (rank + vdim) * 2, flops=2 * T * H * vdim * rank))
             pairs = sum(nq * (nk - nq) + nq * (nq + 1) // 2 for nq, nk in zip(n_qs, n_ks))
             singles = int(max(n_qs) == 1)
-            att = lambda qq, kk, vd, sk: ops.attn_scoremod_paged(qq, kk, kk[..., :vd], ctx.cu_seqlens_q, ctx.cu_seqlens_k, ctx.block_tables,
-                                                                 0.1, 0.0, sk, None, max(n_qs), max(n_ks), singles)
+            meta = (ctx.cu_seqlens_q, ctx.cu_seqlens_k, ctx.block_tables, 0.1)
+            att = lambda qq, kk, vd, sk: ops.attn_latent_paged(qq, kk, kk[..., :vd], *meta, sk, max(n_qs), max(n_ks), singles)
+            old = lambda qq, kk, vd, sk: ops.attn_scoremod_paged(qq, kk, kk[..., :vd], *meta, 0.0, sk, None, max(n_qs), max(n_ks), singles)
             qa, qb = rn(T, H, rank), rn(T, H, lr + lR)
             spec = lambda d, v: dict(nbytes=sum(n_ks) * d * 2 + T * H * (d + v) * 2 if singles else None, flops=2 * (d + v) * H * pairs)
             both(rec, "latent attention with a sink (key %d, value %d)" % (rank, rank), lambda: att(qa, kc, rank, sink),
                  "Benarax latent attention (key %d, value %d)" % (lr + lR, lr), lambda: att(qb, kc2, lr, None), spec(rank, rank),
-                 spec(lr + lR, lr), iters=5)
+                 spec(lr + lR, lr), iters=10)
+            rec["like: the general paged attention launch on the same rows"] = rate(timed(lambda: old(qa, kc, rank, sink), 5), **spec(rank, rank))
             nv.set_context(None)
             out["attention rank %d, %s" % (rank, name)] = rec
 
