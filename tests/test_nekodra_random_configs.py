@@ -53,10 +53,12 @@ def test_random_configuration(seed, backend):
     ck = random_checkpoint(cfg, seed=100 + seed, correction=seed % 5 != 1)
     g = torch.Generator().manual_seed(seed)
     V = cfg["vocab"]
-    p = {"a": torch.randint(0, V, (29,), generator=g).tolist(), "b": torch.randint(0, V, (7,), generator=g).tolist(),
-         "c": torch.randint(0, V, (40,), generator=g).tolist()}
-    portions = {"a": [6, 1, 1, 14, 2, 1], "b": [1], "c": [2, 3, 30, 1]}
-    got = replay(make_engine(cfg, ck, dev, dtype, block_size=4, num_blocks=40, max_seqs=3), p, portions, order={"b": 2, "c": 1})
+    # every second one on pages of 64 (which the matrix-core attention takes) and, where the positions allow it, longer
+    block, more = (64, 4 if cfg["max_positions"] > 64 else 1) if seed % 2 else (4, 1)
+    p = {"a": torch.randint(0, V, (29 * more,), generator=g).tolist(), "b": torch.randint(0, V, (7 * more,), generator=g).tolist(),
+         "c": torch.randint(0, V, (40 * more,), generator=g).tolist()}
+    portions = {"a": [6 * more, 1, 1, 14 * more, 2, 1], "b": [1], "c": [2, 3, 30 * more, 1]}
+    got = replay(make_engine(cfg, ck, dev, dtype, block_size=block, num_blocks=40, max_seqs=3), p, portions, order={"b": 2, "c": 1})
     # Per position, against what the oracle's own bfloat16 evaluation loses there.  float32: every position within 1e-4, or
     # within 2 % of that loss where it is large.  bfloat16: a fault moves most positions, rounding (two experts with almost
     # equal scores) moves a few by more than three times the oracle's loss.
