@@ -1504,6 +1504,10 @@ def attn_latent_paged(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Ten
     Dv = v_cache.shape[3]
     if not (q.dtype == _BF16 and G == 1 and v_cache.data_ptr() == k_cache.data_ptr() and q.is_contiguous() and scale > 0
             and max_seqlen_q > 0 and max_seqlen_k > 0 and dll.nv_attn_latent_ok(D, Dv, bs)):
+        if Dv > 512:                       # the general launch takes up to 512 value columns: the wider ones in turn
+            cuts = [attn_latent_paged(q, k_cache, v_cache[..., c:c + 512], cu_seqlens_q, cu_seqlens_k, block_tables, scale, sink,
+                                      max_seqlen_q, max_seqlen_k, single_rows).view(T, H, -1) for c in range(0, Dv, 512)]
+            return torch.cat(cuts, dim=2).view(T, H * Dv)
         return attn_scoremod_paged(q, k_cache, v_cache, cu_seqlens_q, cu_seqlens_k, block_tables, scale, 0.0, sink, None,
                                    max_seqlen_q, max_seqlen_k, single_rows)
     _need(q.is_cuda and k_cache.is_cuda and k_cache.is_contiguous() and k_cache.dtype == q.dtype and k_cache.shape[3] == D

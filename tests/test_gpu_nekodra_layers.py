@@ -106,7 +106,7 @@ N_Q, N_K = [5, 1, 70, 2, 1], [5, 140, 90, 2, 9]
 
 
 @pytest.mark.parametrize("H,rank,own", [(3, 18, True), (5, 64, True), (16, 128, True), (2, 256, True), (1, 512, True), (9, 40, True),
-                                        (20, 96, False), (4, 7, True), (33, 32, False)])
+                                        (20, 96, False), (4, 7, True), (33, 32, False), (2, 640, True)])
 def test_latent_attention_with_a_sink(dt, H, rank, own):
     ctx, _ = paged_context(N_Q, N_K, 8, 60, 1, DEV)
     nv.set_context(ctx)
