@@ -455,6 +455,64 @@ NV_API int nv_attn_latent_paged(const void* q, const void* cache, void* out, con
                                 float scale, const float* sink, int max_seqlen_q, int max_seqlen_k, int single_rows,
                                 void* workspace, int64_t workspace_bytes, void* stream);
 
+/*
+ * Selective scan, state [num_slots, C, N] fp32 carried per sequence (channels x states):
+ *   dt = softplus(dt_raw + dt_bias);  S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n;  y_c = sum_n S[c, n] C_n + D_c x_c
+ *   out_c = y_c * silu(z_c)
+ * x, dt_raw, z, out: [T, C], Bm, Cm: [T, N] of dtype with row strides; dt_bias, D: [C], A: [C, N] fp32 (A is negative).
+ * N <= 256.  max_seqlen_q: the most rows a sequence has in the step; a step with few sequences is cut into segments along
+ * time through a workspace of nv_selective_scan_workspace_bytes.
+ */
+NV_API int64_t nv_selective_scan_workspace_bytes(int num_seqs, int C, int N, int max_seqlen_q);
+NV_API int nv_selective_scan(const void* x, int64_t x_stride, const void* dt_raw, int64_t dt_stride, const void* z,
+                             int64_t z_stride, const void* Bm, int64_t b_stride, const void* Cm, int64_t c_stride,
+                             const float* dt_bias, const float* A, const float* D, float* state, void* out,
+                             int64_t out_stride, const int32_t* cu_seqlens_q, const int32_t* cu_seqlens_k,
+                             const int32_t* state_slots, int num_seqs, int C, int N, int max_seqlen_q, int dtype,
+                             void* workspace, int64_t workspace_bytes, void* stream);
+
+/*
+ * Linear attention with one constant decay per head, state [num_slots, H, Dk, Dv] fp32 carried per sequence:
+ *   S <- decay_h S + silu(k) silu(v)^T;  o = S^T silu(q)              (out: [T, H * Dv] fp32 with a row stride)
+ * q, k: [T, H * Dk]; v: [T, H * Dv] of dtype with row strides; decay: [H] fp32.  Dk, Dv <= 256.  max_seqlen_q / min_seqlen_q:
+ * the most and fewest rows a sequence has in the step (min_seqlen_q 0: not known); long portions of bf16 rows with Dk <= 128
+ * run in chunks on the matrix cores, through a workspace when a step with few sequences is cut into segments along time.
+ */
+NV_API int64_t nv_fixed_decay_workspace_bytes(int num_seqs, int H, int Dk, int Dv, int max_seqlen_q, int dtype);
+NV_API int nv_fixed_decay_memory(const void* q, const void* k, const void* v, int64_t q_stride, int64_t k_stride,
+                                 int64_t v_stride, const float* decay, float* state, float* out, int64_t out_stride,
+                                 const int32_t* cu_seqlens_q, const int32_t* cu_seqlens_k, const int32_t* state_slots,
+                                 int num_seqs, int H, int Dk, int Dv, int max_seqlen_q, int min_seqlen_q, int dtype,
+                                 void* workspace, int64_t workspace_bytes, void* stream);
+
+/*
+ * In front of nv_attn_scoremod_paged: q [T, H * D] and k [T, G * D] are RMS-normed over the whole row (one weight per column),
+ * rotated on the first rot_dims dimensions of every head (pair (i, i + rot_dims/2) by position * freq[i], cos and sin times
+ * magnitude); q_out [T, H, D] contiguous, k and v [T, G * Dv] scattered into the paged caches (slot < 0: skipped).
+ */
+NV_API int nv_row_norm_rope_store(const void* q, const void* k, const void* v, int64_t q_stride, int64_t k_stride,
+                                  int64_t v_stride, const float* q_norm, const float* k_norm, float eps, const float* freq,
+                                  int rot_dims, float magnitude, const int64_t* positions, const int32_t* slot_mapping,
+                                  void* q_out, void* k_cache, void* v_cache, int dtype, int64_t T, int H, int G, int D,
+                                  int Dv, void* stream);
+
+/*
+ * Outputs of an attention and of a linear memory on their way into one output product, y [rows, H * Dv + cols] contiguous:
+ *   y[:, :H Dv] = left_scale * sigmoid(head_gate[h]) * attn[h];   y[:, H Dv:] = right_scale * sigmoid(gate) * rmsnorm(mem) * norm_w
+ * attn [rows, H * Dv], head_gate [rows, H], gate [rows, cols] of dtype, mem [rows, cols] fp32, all with row strides.
+ */
+NV_API int nv_join_gated(const void* attn, int64_t attn_stride, const void* head_gate, int64_t head_gate_stride, int H, int Dv,
+                         float left_scale, const float* mem, int64_t mem_stride, const float* norm_w, const void* gate,
+                         int64_t gate_stride, int cols, float eps, float right_scale, void* y, int dtype, int64_t rows,
+                         void* stream);
+
+/* y[r, j] = g sigmoid(alpha g) (u + shift), g = min(x[r, j], limit), u = clamp(x[r, inter + j], -limit, limit). */
+NV_API int nv_clamped_glu_rows(const void* x, int64_t x_stride, void* y, int dtype, int64_t rows, int inter, float limit,
+                               float alpha, float shift, void* stream);
+
+/* y[i] = cap * tanh(scale * x[i] / cap) in fp32 for n contiguous elements of dtype (cap 0: scale * x[i]). */
+NV_API int nv_scale_softcap(const void* x, float* y, int dtype, int64_t n, float scale, float cap, void* stream);
+
 #ifdef __cplusplus
 }
 #endif

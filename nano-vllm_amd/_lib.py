@@ -12,7 +12,7 @@ import threading
 _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_HERE, "lib", "libnanovllm_hip.so")
 MIXERS_LIB_PATH = os.path.join(_HERE, "lib", "libnanovllm_hip_mixers.so")
-ABI_VERSION = 12
+ABI_VERSION = 13
 
 _vp, _i32, _i64, _f32 = C.c_void_p, C.c_int, C.c_int64, C.c_float
 
@@ -139,6 +139,18 @@ MIXERS_PROTOTYPES = {
     "nv_attn_latent_workspace_bytes": (_i64, [_i32, _i64, _i32, _i32, _i32, _i32, _i32]),
     "nv_attn_latent_paged": (_i32, [_vp, _vp, _vp, _vp, _vp, _vp, _i32, _i32, _i64, _i32, _i32, _i32, _i64, _i32, _f32, _vp, _i32,
                                     _i32, _i32, _vp, _i64, _vp]),
+    "nv_selective_scan_workspace_bytes": (_i64, [_i32, _i32, _i32, _i32]),
+    "nv_selective_scan": (_i32, [_vp, _i64, _vp, _i64, _vp, _i64, _vp, _i64, _vp, _i64, _vp, _vp, _vp, _vp, _vp, _i64, _vp, _vp,
+                                 _vp, _i32, _i32, _i32, _i32, _i32, _vp, _i64, _vp]),
+    "nv_fixed_decay_workspace_bytes": (_i64, [_i32, _i32, _i32, _i32, _i32, _i32]),
+    "nv_fixed_decay_memory": (_i32, [_vp, _vp, _vp, _i64, _i64, _i64, _vp, _vp, _vp, _i64, _vp, _vp, _vp, _i32, _i32, _i32, _i32,
+                                     _i32, _i32, _i32, _vp, _i64, _vp]),
+    "nv_row_norm_rope_store": (_i32, [_vp, _vp, _vp, _i64, _i64, _i64, _vp, _vp, _f32, _vp, _i32, _f32, _vp, _vp, _vp, _vp, _vp,
+                                      _i32, _i64, _i32, _i32, _i32, _i32, _vp]),
+    "nv_join_gated": (_i32, [_vp, _i64, _vp, _i64, _i32, _i32, _f32, _vp, _i64, _vp, _vp, _i64, _i32, _f32, _f32, _vp, _i32, _i64,
+                             _vp]),
+    "nv_clamped_glu_rows": (_i32, [_vp, _i64, _vp, _i32, _i64, _i32, _f32, _f32, _f32, _vp]),
+    "nv_scale_softcap": (_i32, [_vp, _vp, _i32, _i64, _f32, _f32, _vp]),
     "nv_moe_up_relu2": (_i32, [_vp, _i64, _vp, _vp, _vp, _vp, _i32, _i64, _i32, _i32, _i32, _i32, _i32, _vp]),
 }
 DTYPE_BF16, DTYPE_F32 = 0, 1

@@ -1,6 +1,6 @@
 // Linear recurrences whose memory is written BEFORE it is read, state [Dk, Dv] (key channel x value channel) in fp32
 // per head, carried per SEQUENCE in numbered slots (a sequence whose rows start at position 0 starts from a zero state
-// whatever its slot holds).  Two forms share one kernel; both are  S <- diag(w) S + k v^T,  o = S^T r  with per-token
+// whatever its slot holds).  Three forms share one kernel; all are  S <- diag(w) S + k v^T,  o = S^T r  with per-token
 // vectors w, k, r [Dk] made from the raw projections in fp32:
 //
 //   nv_mlstm_memory        (matrix memory with exponential gates and a running maximum that keeps them bounded)
@@ -14,6 +14,9 @@
 //       f = lower + (1 - lower) sigmoid(f_raw + b_f)   per head and key channel;   w = f;   k = 1 - f;   r = silu(q_raw)
 //       out = o / sqrt(mean(o^2) + eps) * norm_w        (one weight [Dv] for all heads)
 //
+//   fixed form             (one constant decay per head; fixed_decay.hip takes long portions and owns the entry point)
+//       w = decay[h];   k = silu(k_raw);   v = silu(v_raw);   r = silu(q_raw);   out = o in fp32
+//
 // Layout as in the decayed-memory kernel next door: one workgroup per (sequence, head); a lane owns one value column
 // and a quarter of the key rows (its quad index q owns rows q * RPL .. q * RPL + RPL - 1, read from LDS four at a time,
 // the four runs RPL + 4 words apart so that a quad's 16-byte reads fall on different banks), so the state lives in
@@ -22,14 +25,17 @@
 // every exponential around it is taken in parallel), each wave then runs those tokens for its 16 columns, and the
 // tile's output is normalised and written by all waves.
 #include <algorithm>
+#include <type_traits>
 
-#include "nv_common.h"
+#include "fixed_decay.h"
 #include "../../include/nanovllm_hip_mixers.h"
 
 namespace nv {
 
 constexpr int kGmMaxTile = 16;
 constexpr int kGmLdsBudget = 60 * 1024;
+
+enum { kGmMatrix = 0, kGmWrite = 1, kGmFixed = 2 };
 
 __device__ __forceinline__ float gm_sigmoid(float x) { return 1.0f / (1.0f + expf(-x)); }
 __device__ __forceinline__ float gm_logsigmoid(float x) { return fminf(x, 0.f) - log1pf(expf(-fabsf(x))); }
@@ -60,10 +66,14 @@ struct GmArgs {
     int H, Dk, Dv;
     float eps, cap, q_scale;
     int tile;
+    const float* decay;                    // fixed form: [H]
+    float* out32;                          // fixed form: [T, H * Dv]
+    int max_rows;                          // fixed form: sequences with more rows in the step are left to another launch (0: none)
 };
 
-template <typename T, int RPL, bool MATRIX, int MAXT>
+template <typename T, int RPL, int FORM, int MAXT>
 __global__ __launch_bounds__(MAXT) void gated_memory_kernel(const GmArgs<T> a) {
+    constexpr bool MATRIX = FORM == kGmMatrix;
     constexpr int DP = (RPL + 4) * 4;                 // LDS words per token and vector: four runs of RPL rows, padded
     constexpr int NPL = (4 * RPL + 63) / 64;          // key channels a lane of wave 0 owns for the vector n
     extern __shared__ float smem[];
@@ -80,6 +90,8 @@ __global__ __launch_bounds__(MAXT) void gated_memory_kernel(const GmArgs<T> a) {
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, n_waves = blockDim.x >> 6;
     const int q0 = a.cu_q[b], len_q = a.cu_q[b + 1] - q0;
     if (len_q <= 0) return;
+    if constexpr (FORM == kGmFixed)
+        if (a.max_rows > 0 && len_q > a.max_rows) return;
     const int start = (a.cu_k[b + 1] - a.cu_k[b]) - len_q;
     const int col = wave * 16 + (lane >> 2), q = lane & 3;
     const bool live = col < Dv;
@@ -139,6 +151,11 @@ __global__ __launch_bounds__(MAXT) void gated_memory_kernel(const GmArgs<T> a) {
                     wv = gf[tt];
                     kv = gi[tt] * (float)a.k[t * a.k_stride + hd];
                     rv = qv * a.q_scale;
+                } else if constexpr (FORM == kGmFixed) {
+                    const float kr = (float)a.k[t * a.k_stride + hd];
+                    wv = a.decay[h];
+                    kv = kr / (1.0f + expf(-kr));
+                    rv = qv / (1.0f + expf(-qv));
                 } else {
                     const float lo = a.lower[hd];
                     wv = lo + (1.0f - lo) * gm_sigmoid((float)a.f_raw[t * a.f_stride + hd] + a.f_bias[hd]);
@@ -152,7 +169,9 @@ __global__ __launch_bounds__(MAXT) void gated_memory_kernel(const GmArgs<T> a) {
         }
         for (int i = tid; i < nt * Dv; i += blockDim.x) {
             const int tt = i / Dv, c = i % Dv;
-            vs[tt * Dv + c] = (float)a.v[(int64_t)(q0 + t0 + tt) * a.v_stride + (int64_t)h * Dv + c];
+            float vv = (float)a.v[(int64_t)(q0 + t0 + tt) * a.v_stride + (int64_t)h * Dv + c];
+            if constexpr (FORM == kGmFixed) vv = vv / (1.0f + expf(-vv));
+            vs[tt * Dv + c] = vv;
         }
         __syncthreads();
         if constexpr (MATRIX) {
@@ -198,6 +217,11 @@ __global__ __launch_bounds__(MAXT) void gated_memory_kernel(const GmArgs<T> a) {
         }
         __syncthreads();
         // ---- the tile's output ---------------------------------------------------------------------------
+        if constexpr (FORM == kGmFixed) {
+            for (int i = tid; i < nt * Dv; i += blockDim.x)
+                a.out32[(int64_t)(q0 + t0 + i / Dv) * a.out_stride + (int64_t)h * Dv + i % Dv] = os[i];
+            continue;
+        }
         for (int tt = wave; tt < nt; tt += n_waves) {
             const int64_t t = q0 + t0 + tt;
             const float inv_den = MATRIX ? 1.0f / gm[tt] : 1.0f;
@@ -235,7 +259,7 @@ __global__ __launch_bounds__(MAXT) void gated_memory_kernel(const GmArgs<T> a) {
     }
 }
 
-template <typename T, bool MATRIX>
+template <typename T, int FORM>
 static int launch_gated_memory(GmArgs<T> a, int B, hipStream_t s, const char* what) {
     const int waves = (a.Dv + 15) / 16;
     const dim3 grid((unsigned)B, (unsigned)a.H), block((unsigned)waves * 64);
@@ -245,9 +269,9 @@ static int launch_gated_memory(GmArgs<T> a, int B, hipStream_t s, const char* wh
     const size_t smem = per_token * a.tile;
 #define NV_GM_CASE(R)                                                                                            \
     case R:                                                                                                      \
-        if (waves <= 4) hipLaunchKernelGGL((gated_memory_kernel<T, R, MATRIX, 256>), grid, block, smem, s, a);       \
-        else if (waves <= 8) hipLaunchKernelGGL((gated_memory_kernel<T, R, MATRIX, 512>), grid, block, smem, s, a);  \
-        else hipLaunchKernelGGL((gated_memory_kernel<T, R, MATRIX, 1024>), grid, block, smem, s, a);                 \
+        if (waves <= 4) hipLaunchKernelGGL((gated_memory_kernel<T, R, FORM, 256>), grid, block, smem, s, a);       \
+        else if (waves <= 8) hipLaunchKernelGGL((gated_memory_kernel<T, R, FORM, 512>), grid, block, smem, s, a);  \
+        else hipLaunchKernelGGL((gated_memory_kernel<T, R, FORM, 1024>), grid, block, smem, s, a);                 \
         break;
     switch (rpl) {
         NV_GM_CASE(8)
@@ -258,6 +282,32 @@ static int launch_gated_memory(GmArgs<T> a, int B, hipStream_t s, const char* wh
     }
 #undef NV_GM_CASE
     return check_launch(what);
+}
+
+int launch_fixed_decay_rows(const FixedDecayArgs& f, int dtype, int max_rows, hipStream_t s) {
+    auto fill = [&](auto* none) {
+        using T = std::remove_pointer_t<decltype(none)>;
+        GmArgs<T> a{};
+        a.q = (const T*)f.q;
+        a.k = (const T*)f.k;
+        a.v = (const T*)f.v;
+        a.q_stride = f.q_stride;
+        a.k_stride = f.k_stride;
+        a.v_stride = f.v_stride;
+        a.state = f.state;
+        a.out_stride = f.out_stride;
+        a.cu_q = f.cu_q;
+        a.cu_k = f.cu_k;
+        a.slots = f.slots;
+        a.H = f.H;
+        a.Dk = f.Dk;
+        a.Dv = f.Dv;
+        a.decay = f.decay;
+        a.out32 = f.out;
+        a.max_rows = max_rows;
+        return launch_gated_memory<T, kGmFixed>(a, f.num_seqs, s, "nv_fixed_decay_memory");
+    };
+    return dtype == NV_DTYPE_BF16 ? fill((__bf16*)nullptr) : fill((float*)nullptr);
 }
 
 }  // namespace nv
@@ -284,14 +334,14 @@ extern "C" int nv_mlstm_memory(const void* q, const void* k, const void* v, int6
         GmArgs<__bf16> a{(const __bf16*)q, (const __bf16*)k, (const __bf16*)v, q_stride, k_stride, v_stride, nullptr, 0,
                          i_pre, f_pre, gate_pre_stride, (const __bf16*)gate_raw, gate_stride, i_bias, f_bias, nullptr,
                          norm_w, Dv, state, norm_state, max_state, (__bf16*)out, out_stride, cu_seqlens_q, cu_seqlens_k,
-                         state_slots, H, Dk, Dv, eps, gate_cap, q_scale, 0};
-        return launch_gated_memory<__bf16, true>(a, num_seqs, s, "nv_mlstm_memory");
+                         state_slots, H, Dk, Dv, eps, gate_cap, q_scale, 0, nullptr, nullptr, 0};
+        return launch_gated_memory<__bf16, kGmMatrix>(a, num_seqs, s, "nv_mlstm_memory");
     }
     GmArgs<float> a{(const float*)q, (const float*)k, (const float*)v, q_stride, k_stride, v_stride, nullptr, 0, i_pre,
                     f_pre, gate_pre_stride, (const float*)gate_raw, gate_stride, i_bias, f_bias, nullptr, norm_w, Dv,
                     state, norm_state, max_state, (float*)out, out_stride, cu_seqlens_q, cu_seqlens_k, state_slots, H, Dk,
-                    Dv, eps, gate_cap, q_scale, 0};
-    return launch_gated_memory<float, true>(a, num_seqs, s, "nv_mlstm_memory");
+                    Dv, eps, gate_cap, q_scale, 0, nullptr, nullptr, 0};
+    return launch_gated_memory<float, kGmMatrix>(a, num_seqs, s, "nv_mlstm_memory");
 }
 
 extern "C" int nv_gated_write_memory(const void* q, const void* f_raw, const void* v, int64_t q_stride, int64_t f_stride,
@@ -311,11 +361,11 @@ extern "C" int nv_gated_write_memory(const void* q, const void* f_raw, const voi
     if (dtype == NV_DTYPE_BF16) {
         GmArgs<__bf16> a{(const __bf16*)q, nullptr, (const __bf16*)v, q_stride, 0, v_stride, (const __bf16*)f_raw, f_stride,
                          nullptr, nullptr, 0, nullptr, 0, nullptr, f_bias, lower, norm_w, 0, state, nullptr, nullptr,
-                         (__bf16*)out, out_stride, cu_seqlens_q, cu_seqlens_k, state_slots, H, Dk, Dv, eps, 0.f, 1.f, 0};
-        return launch_gated_memory<__bf16, false>(a, num_seqs, s, "nv_gated_write_memory");
+                         (__bf16*)out, out_stride, cu_seqlens_q, cu_seqlens_k, state_slots, H, Dk, Dv, eps, 0.f, 1.f, 0, nullptr, nullptr, 0};
+        return launch_gated_memory<__bf16, kGmWrite>(a, num_seqs, s, "nv_gated_write_memory");
     }
     GmArgs<float> a{(const float*)q, nullptr, (const float*)v, q_stride, 0, v_stride, (const float*)f_raw, f_stride, nullptr,
                     nullptr, 0, nullptr, 0, nullptr, f_bias, lower, norm_w, 0, state, nullptr, nullptr, (float*)out,
-                    out_stride, cu_seqlens_q, cu_seqlens_k, state_slots, H, Dk, Dv, eps, 0.f, 1.f, 0};
-    return launch_gated_memory<float, false>(a, num_seqs, s, "nv_gated_write_memory");
+                    out_stride, cu_seqlens_q, cu_seqlens_k, state_slots, H, Dk, Dv, eps, 0.f, 1.f, 0, nullptr, nullptr, 0};
+    return launch_gated_memory<float, kGmWrite>(a, num_seqs, s, "nv_gated_write_memory");
 }

@@ -1,0 +1,352 @@
+// Selective scan: a diagonal linear recurrence per channel whose decay and input depend on the token, state [C, N] (channel
+// x state) in fp32, carried per SEQUENCE in numbered slots (a sequence whose rows start at position 0 starts from a zero
+// state whatever its slot holds):
+//
+//   dt = softplus(dt_raw + dt_bias)                                       one per token and channel
+//   S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n;   y_c = sum_n S[c, n] C_n + D_c x_c
+//   out_c = y_c * silu(z_c)
+//
+// B and C are vectors [N] per token shared by all channels.  Everything behind the raw inputs is fp32.
+//
+// Layout: L lanes share a channel and own SPL of its states each, in registers; a workgroup of 256 threads takes 256 / L
+// channels of one sequence.  16 tokens at a time are prepared into LDS (softplus and dt x once per token and channel, B and
+// C once per token), the next 16 tokens' inputs being on their way into registers meanwhile; the token loop has no
+// barrier: two small LDS reads per vector, one exponential and three multiply-adds per state, a sum over the L lanes.
+//
+// A step with too few (sequence, channel) pairs to fill the chip is cut into segments along time: a first launch runs every
+// segment but a sequence's last from a zero state and leaves its end state and its sum of dt per channel (the decay of a
+// whole segment is exp(A * sum dt)); in the second launch a segment folds what is in front of it into its start state and
+// runs as usual.
+#include <algorithm>
+
+#include "row_pieces.h"
+#include "../../include/nanovllm_hip_mixers.h"
+
+namespace nv {
+
+constexpr int kScThreads = 256;
+constexpr int kScTile = 16;                    // tokens prepared at a time
+
+__device__ __forceinline__ float sc_softplus(float x) { return x > 20.f ? x : log1pf(expf(x)); }
+__device__ __forceinline__ float sc_silu(float x) { return x / (1.0f + expf(-x)); }
+
+// Sum over aligned groups of L lanes; every lane of the group gets it.
+template <int L>
+__device__ __forceinline__ float sc_group_sum(float x) {
+    if constexpr (L >= 2) x += dpp_f32<0xB1>(x);      // quad_perm [1,0,3,2]
+    if constexpr (L >= 4) x += dpp_f32<0x4E>(x);      // quad_perm [2,3,0,1]
+    if constexpr (L >= 8) x += dpp_f32<0x141>(x);     // row_half_mirror
+    if constexpr (L >= 16) x += dpp_f32<0x140>(x);    // row_mirror
+    if constexpr (L >= 32) x += __shfl_xor(x, 16);
+    if constexpr (L >= 64) x += __shfl_xor(x, 32);
+    return x;
+}
+
+template <typename T>
+struct ScArgs {
+    const T *x, *dt_raw, *z, *Bm, *Cm;         // [T, C], [T, C], [T, C], [T, N], [T, N] with row strides
+    int64_t x_stride, dt_stride, z_stride, b_stride, c_stride;
+    const float *dt_bias, *A, *D;              // [C], [C, N], [C]
+    float* state;                              // [slots, C, N]
+    T* out;                                    // [T, C]
+    int64_t out_stride;
+    const int *cu_q, *cu_k, *slots;
+    int C, N;
+    int seg_len, nseg;                         // tokens per segment (a multiple of kScTile), segments of the longest sequence
+    float *seg_state, *seg_dt;                 // [B, nseg, C, N], [B, nseg, C]
+    int vec;                                   // rows of x, dt_raw, z, out may be walked in pieces of four columns
+};
+
+// Four neighbouring columns of a row, zeros from `cols` on.
+template <typename T>
+__device__ __forceinline__ Cols<4> sc_load4(const T* row, int c, int cols, bool vec) {
+    if (vec) return row_load<4>(row + c);
+    Cols<4> o;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) o.v[e] = c + e < cols ? (float)row[c + e] : 0.f;
+    return o;
+}
+
+enum { kScWhole = 0, kScSummary = 1, kScFinal = 2 };
+
+template <typename T, int L, int SPL, int MODE>
+__global__ __launch_bounds__(kScThreads) void selective_scan_kernel(const ScArgs<T> a) {
+    constexpr int CPB = kScThreads / L;                          // channels of the workgroup
+    constexpr int NP = L * SPL;                                  // states, padded
+    constexpr int PIECES = kScTile * CPB / 4;                    // four-channel pieces of a tile
+    constexpr int IT = (PIECES + kScThreads - 1) / kScThreads;
+    constexpr int IB = (kScTile * NP + kScThreads - 1) / kScThreads;
+    __shared__ float2 dts[kScTile][CPB];                         // (dt, dt x)
+    __shared__ float bs[kScTile][NP], cs[kScTile][NP];
+    __shared__ float ys[kScTile][CPB];
+    const int b = blockIdx.x, c0 = blockIdx.y * CPB, seg = blockIdx.z;
+    const int q0 = a.cu_q[b], len_q = a.cu_q[b + 1] - q0;
+    if (len_q <= 0) return;
+    const int first = seg * a.seg_len, last_seg = min((len_q - 1) / a.seg_len, a.nseg - 1);
+    if (seg > last_seg) return;
+    const int start = (a.cu_k[b + 1] - a.cu_k[b]) - len_q;
+    const int tid = threadIdx.x, ch = tid / L, sub = tid % L;
+    const int C = a.C, N = a.N, c = c0 + ch;
+    const bool live = c < C;
+    float* slot_state = a.state + ((int64_t)a.slots[b] * C + c) * N;
+    float A2[SPL], S[SPL];                                       // A log2(e); the state
+#pragma unroll
+    for (int i = 0; i < SPL; ++i) {
+        const int n = sub * SPL + i;
+        const bool in = live && n < N;
+        A2[i] = in ? a.A[(int64_t)c * N + n] * 1.4426950408889634f : 0.f;
+        S[i] = 0.f;
+    }
+    if constexpr (MODE == kScSummary) {
+        if (last_seg == 0) return;                               // nobody folds
+        if (seg == last_seg) {                                   // the start state is handed on from here: the second launch
+            float* dst = a.seg_state + (((int64_t)b * a.nseg + seg) * C + c) * N;      // overwrites the slot
+#pragma unroll
+            for (int i = 0; i < SPL; ++i) {
+                const int n = sub * SPL + i;
+                if (live && n < N) dst[n] = start > 0 ? slot_state[n] : 0.f;
+            }
+            return;
+        }
+    } else {
+        const float* src = slot_state;
+        bool have = start > 0;
+        if constexpr (MODE == kScFinal) {
+            if (last_seg > 0) {
+                src = a.seg_state + (((int64_t)b * a.nseg + last_seg) * C + c) * N;
+                have = true;
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < SPL; ++i) {
+            const int n = sub * SPL + i;
+            if (have && live && n < N) S[i] = src[n];
+        }
+        if constexpr (MODE == kScFinal) {
+            for (int s = 0; s < seg; ++s) {
+                const int64_t at = ((int64_t)b * a.nseg + s) * C + c;
+                const float dsum = live ? a.seg_dt[at] : 0.f;
+#pragma unroll
+                for (int i = 0; i < SPL; ++i) {
+                    const int n = sub * SPL + i;
+                    if (live && n < N) S[i] = __builtin_amdgcn_exp2f(dsum * A2[i]) * S[i] + a.seg_state[at * N + n];
+                }
+            }
+        }
+    }
+    float dt_sum = 0.f;
+    const int stop = seg == last_seg ? len_q : first + a.seg_len;
+    // registers of the tile that comes next, and (x, z) of the one that is being scanned
+    Cols<4> ndt[IT], nx[IT], nz[IT], x_cur[IT], z_cur[IT];
+    float nb[IB], nc[IB];
+    auto fetch = [&](int t0) {
+#pragma unroll
+        for (int k = 0; k < IT; ++k) {
+            const int p = tid + k * kScThreads, tt = p / (CPB / 4), cc = c0 + (p % (CPB / 4)) * 4;
+            if (p < PIECES && t0 + tt < stop && cc < C) {
+                const int64_t t = q0 + t0 + tt;
+                ndt[k] = sc_load4(a.dt_raw + t * a.dt_stride, cc, C, a.vec);
+                nx[k] = sc_load4(a.x + t * a.x_stride, cc, C, a.vec);
+                if constexpr (MODE != kScSummary) nz[k] = sc_load4(a.z + t * a.z_stride, cc, C, a.vec);
+            } else {
+#pragma unroll
+                for (int e = 0; e < 4; ++e) ndt[k].v[e] = nx[k].v[e] = nz[k].v[e] = 0.f;
+            }
+        }
+#pragma unroll
+        for (int k = 0; k < IB; ++k) {
+            const int p = tid + k * kScThreads, tt = p / NP, n = p % NP;
+            const bool in = tt < kScTile && t0 + tt < stop && n < N;
+            nb[k] = in ? (float)a.Bm[(int64_t)(q0 + t0 + tt) * a.b_stride + n] : 0.f;
+            if constexpr (MODE != kScSummary) nc[k] = in ? (float)a.Cm[(int64_t)(q0 + t0 + tt) * a.c_stride + n] : 0.f;
+        }
+    };
+    fetch(first);
+    for (int t0 = first; t0 < stop; t0 += kScTile) {
+        const int nt = min(kScTile, stop - t0);
+        __syncthreads();                                         // the previous tile has been scanned and written
+#pragma unroll
+        for (int k = 0; k < IT; ++k) {
+            const int p = tid + k * kScThreads, tt = p / (CPB / 4), cl = (p % (CPB / 4)) * 4;
+            x_cur[k] = nx[k];
+            z_cur[k] = nz[k];
+            if (p < PIECES) {
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    // (dt = 0 behind the portion's end: those steps leave the state as it is)
+                    const float dt = tt < nt && c0 + cl + e < C ? sc_softplus(ndt[k].v[e] + a.dt_bias[c0 + cl + e]) : 0.f;
+                    dts[tt][cl + e] = make_float2(dt, dt * nx[k].v[e]);
+                }
+            }
+        }
+#pragma unroll
+        for (int k = 0; k < IB; ++k) {
+            const int p = tid + k * kScThreads, tt = p / NP, n = p % NP;
+            if (tt < kScTile) {
+                bs[tt][n] = nb[k];
+                if constexpr (MODE != kScSummary) cs[tt][n] = nc[k];
+            }
+        }
+        __syncthreads();
+        if (t0 + kScTile < stop) fetch(t0 + kScTile);
+        // ---- the recurrence over the tile, no barrier inside ---------------------------------------------
+        for (int t4 = 0; t4 < nt; t4 += 4) {                     // four tokens at a time: their exponentials overlap
+            float y[4];
+#pragma unroll
+            for (int u = 0; u < 4; ++u) {
+                const float2 d = dts[t4 + u][ch];
+                const float* bt = &bs[t4 + u][sub * SPL];
+                const float* ct = &cs[t4 + u][sub * SPL];
+                y[u] = 0.f;
+#pragma unroll
+                for (int i = 0; i < SPL; ++i) {
+                    S[i] = __builtin_amdgcn_exp2f(d.x * A2[i]) * S[i] + d.y * bt[i];
+                    if constexpr (MODE != kScSummary) y[u] += S[i] * ct[i];
+                }
+                if constexpr (MODE == kScSummary) dt_sum += d.x;
+            }
+            if constexpr (MODE != kScSummary) {
+#pragma unroll
+                for (int u = 0; u < 4; ++u) y[u] = sc_group_sum<L>(y[u]);
+                if (sub == 0) {
+#pragma unroll
+                    for (int u = 0; u < 4; ++u) ys[t4 + u][ch] = y[u];
+                }
+            }
+        }
+        if constexpr (MODE != kScSummary) {
+            __syncthreads();
+#pragma unroll
+            for (int k = 0; k < IT; ++k) {
+                const int p = tid + k * kScThreads, tt = p / (CPB / 4), cl = (p % (CPB / 4)) * 4, cc = c0 + cl;
+                if (p >= PIECES || tt >= nt || cc >= C) continue;
+                Cols<4> o;
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    const float skip = cc + e < C ? a.D[cc + e] : 0.f;
+                    o.v[e] = (ys[tt][cl + e] + skip * x_cur[k].v[e]) * sc_silu(z_cur[k].v[e]);
+                }
+                T* dst = a.out + (int64_t)(q0 + t0 + tt) * a.out_stride + cc;
+                if (a.vec) {
+                    row_store<4>(dst, o);
+                } else {
+#pragma unroll
+                    for (int e = 0; e < 4; ++e)
+                        if (cc + e < C) dst[e] = (T)o.v[e];
+                }
+            }
+        }
+    }
+    if (!live) return;
+    if constexpr (MODE == kScSummary) {
+        const int64_t at = ((int64_t)b * a.nseg + seg) * C + c;
+        if (sub == 0) a.seg_dt[at] = dt_sum;
+#pragma unroll
+        for (int i = 0; i < SPL; ++i) {
+            const int n = sub * SPL + i;
+            if (n < N) a.seg_state[at * N + n] = S[i];
+        }
+    } else if (seg == last_seg) {
+#pragma unroll
+        for (int i = 0; i < SPL; ++i) {
+            const int n = sub * SPL + i;
+            if (n < N) slot_state[n] = S[i];
+        }
+    }
+}
+
+struct ScPlan {
+    int L, SPL, nseg, seg_len;
+    int64_t ws_floats;
+};
+
+// Lanes per channel and states per lane from N; segments so that the launch has about two waves per SIMD.
+static ScPlan sc_plan(int B, int C, int N, int max_seqlen_q) {
+    ScPlan p{1, 4, 1, 0, 0};
+    while (p.L * 4 < N) p.L *= 2;
+    // eight states per lane (half the lanes, less work per token beside the states) when there are plenty of waves
+    if (p.L >= 4 && (int64_t)B * C * p.L / 64 >= 8192) {
+        p.SPL = 8;
+        p.L /= 2;
+    }
+    const int cpb = kScThreads / p.L;
+    const int64_t waves = (int64_t)B * ((C + cpb - 1) / cpb) * (kScThreads / 64);
+    const int mq = std::max(1, max_seqlen_q);
+    p.seg_len = (mq + kScTile - 1) / kScTile * kScTile;
+    if (waves < 1024 && mq >= 256) {
+        const int want = (int)std::min<int64_t>((2048 + waves - 1) / waves, 16);
+        const int most = mq / 128;
+        p.nseg = std::max(1, std::min(want, most));
+        p.seg_len = ((mq + p.nseg - 1) / p.nseg + kScTile - 1) / kScTile * kScTile;
+        p.nseg = (mq + p.seg_len - 1) / p.seg_len;
+    }
+    if (p.nseg > 1) p.ws_floats = (int64_t)B * p.nseg * C * (N + 1);
+    return p;
+}
+
+template <typename T, int L, int SPL>
+static void launch_scan(const ScArgs<T>& a, int B, hipStream_t s) {
+    constexpr int CPB = kScThreads / L;
+    const dim3 grid((unsigned)B, (unsigned)((a.C + CPB - 1) / CPB), (unsigned)a.nseg), block(kScThreads);
+    if (a.nseg == 1) {
+        hipLaunchKernelGGL((selective_scan_kernel<T, L, SPL, kScWhole>), grid, block, 0, s, a);
+        return;
+    }
+    hipLaunchKernelGGL((selective_scan_kernel<T, L, SPL, kScSummary>), grid, block, 0, s, a);
+    hipLaunchKernelGGL((selective_scan_kernel<T, L, SPL, kScFinal>), grid, block, 0, s, a);
+}
+
+template <typename T>
+static int run_scan(const ScArgs<T>& a, const ScPlan& p, int B, hipStream_t s) {
+#define NV_SC(LL, SS) \
+    if (p.L == LL && p.SPL == SS) { launch_scan<T, LL, SS>(a, B, s); return check_launch("nv_selective_scan"); }
+    NV_SC(1, 4) NV_SC(2, 4) NV_SC(4, 4) NV_SC(8, 4) NV_SC(16, 4) NV_SC(32, 4) NV_SC(64, 4)
+    NV_SC(2, 8) NV_SC(4, 8) NV_SC(8, 8) NV_SC(16, 8) NV_SC(32, 8)
+#undef NV_SC
+    set_error("nv_selective_scan: no kernel for %d lanes x %d states", p.L, p.SPL);
+    return NV_ERR_UNSUPPORTED;
+}
+
+}  // namespace nv
+
+extern "C" int64_t nv_selective_scan_workspace_bytes(int num_seqs, int C, int N, int max_seqlen_q) {
+    if (num_seqs <= 0 || C <= 0 || N <= 0 || N > 256) return 0;
+    return nv::sc_plan(num_seqs, C, N, max_seqlen_q).ws_floats * (int64_t)sizeof(float);
+}
+
+extern "C" int nv_selective_scan(const void* x, int64_t x_stride, const void* dt_raw, int64_t dt_stride, const void* z,
+                                 int64_t z_stride, const void* Bm, int64_t b_stride, const void* Cm, int64_t c_stride,
+                                 const float* dt_bias, const float* A, const float* D_skip, float* state, void* out,
+                                 int64_t out_stride, const int32_t* cu_seqlens_q, const int32_t* cu_seqlens_k,
+                                 const int32_t* state_slots, int num_seqs, int C, int N, int max_seqlen_q, int dtype,
+                                 void* workspace, int64_t workspace_bytes, void* stream) {
+    using namespace nv;
+    NV_REQUIRE(num_seqs >= 0 && C > 0 && N > 0 && max_seqlen_q >= 1, NV_ERR_INVALID_ARG, "nv_selective_scan: bad sizes");
+    if (num_seqs == 0) return NV_OK;
+    NV_REQUIRE(x && dt_raw && z && Bm && Cm && dt_bias && A && D_skip && state && out && cu_seqlens_q && cu_seqlens_k &&
+                   state_slots,
+               NV_ERR_INVALID_ARG, "nv_selective_scan: null pointer");
+    NV_REQUIRE(N <= 256, NV_ERR_UNSUPPORTED, "nv_selective_scan: %d states per channel exceed 256", N);
+    NV_REQUIRE(dtype == NV_DTYPE_BF16 || dtype == NV_DTYPE_F32, NV_ERR_INVALID_ARG, "nv_selective_scan: bad dtype");
+    const ScPlan p = sc_plan(num_seqs, C, N, max_seqlen_q);
+    NV_REQUIRE((C + kScThreads / p.L - 1) / (kScThreads / p.L) < 65536, NV_ERR_UNSUPPORTED, "nv_selective_scan: launch too large");
+    NV_REQUIRE(p.ws_floats == 0 || (workspace && workspace_bytes >= p.ws_floats * (int64_t)sizeof(float)), NV_ERR_WORKSPACE,
+               "nv_selective_scan: workspace of %lld bytes, need %lld", (long long)workspace_bytes,
+               (long long)(p.ws_floats * (int64_t)sizeof(float)));
+    hipStream_t s = (hipStream_t)stream;
+    float* seg_state = (float*)workspace;
+    float* seg_dt = p.nseg > 1 ? seg_state + (int64_t)num_seqs * p.nseg * C * N : nullptr;
+    const int align = dtype == NV_DTYPE_BF16 ? 8 : 16;
+    const int vec = C % 4 == 0 && x_stride % 4 == 0 && dt_stride % 4 == 0 && z_stride % 4 == 0 && out_stride % 4 == 0 &&
+                    ((uintptr_t)x | (uintptr_t)dt_raw | (uintptr_t)z | (uintptr_t)out) % align == 0;
+    if (dtype == NV_DTYPE_BF16) {
+        const ScArgs<__bf16> a{(const __bf16*)x, (const __bf16*)dt_raw, (const __bf16*)z, (const __bf16*)Bm, (const __bf16*)Cm,
+                               x_stride, dt_stride, z_stride, b_stride, c_stride, dt_bias, A, D_skip, state, (__bf16*)out,
+                               out_stride, cu_seqlens_q, cu_seqlens_k, state_slots, C, N, p.seg_len, p.nseg, seg_state, seg_dt, vec};
+        return run_scan<__bf16>(a, p, num_seqs, s);
+    }
+    const ScArgs<float> a{(const float*)x, (const float*)dt_raw, (const float*)z, (const float*)Bm, (const float*)Cm, x_stride,
+                          dt_stride, z_stride, b_stride, c_stride, dt_bias, A, D_skip, state, (float*)out, out_stride,
+                          cu_seqlens_q, cu_seqlens_k, state_slots, C, N, p.seg_len, p.nseg, seg_state, seg_dt, vec};
+    return run_scan<float>(a, p, num_seqs, s);
+}

@@ -5,7 +5,8 @@ kernels.
 and a running maximum m that keeps the exponentials bounded (m starts at 0):
     m' = max(f + m, i);  S <- exp(f + m - m') S + exp(i - m') k v^T;  n likewise with k;  o = S^T q / (max(|n . q|, exp(-m')) + 1e-6)
 with i = cap tanh((i_pre + b_i) / cap) and f = logsigmoid(cap tanh((f_pre + b_f) / cap)); the read-out is normalised per
-head, weighted and gated by a sigmoid.  ``GatedWriteMemory``: S <- diag(f) S + (1 - f) v^T, o = S^T silu(q), with
+head, weighted and gated by a sigmoid.  ``FixedDecayMemory``: S <- decay_h S + silu(k) silu(v)^T, o = S^T silu(q), one constant
+decay per head, o in float32 as it is (what norms and gates it spans the heads).  ``GatedWriteMemory``: S <- diag(f) S + (1 - f) v^T, o = S^T silu(q), with
 f = lower + (1 - lower) sigmoid(f_raw + b_f) per head and key channel; the read-out is normalised per head with one
 weight [Dv] for all heads.
 
@@ -61,3 +62,21 @@ class GatedWriteMemory(nn.Module):
         ctx = get_context()
         return ops.gated_write_memory(q, f_raw, v, self.f_bias, self.lower, self.norm_weight, cache["state"],
                                       ctx.cu_seqlens_q, ctx.cu_seqlens_k, ctx.state_slots, self.eps)
+
+
+class FixedDecayMemory(nn.Module):
+    def __init__(self, num_heads: int, key_dim: int, value_dim: int, decay, device=None):
+        super().__init__()
+        self.num_heads, self.key_dim, self.value_dim = num_heads, key_dim, value_dim
+        decay = torch.as_tensor(decay, dtype=torch.float64).to(torch.float32)
+        assert decay.shape == (num_heads,)
+        self.register_buffer("decay", decay.to(device) if device is not None else decay, persistent=False)
+
+    def state_shapes(self) -> dict:
+        return {"state": ((self.num_heads, self.key_dim, self.value_dim), torch.float32)}
+
+    def forward(self, q, k, v, cache: dict) -> torch.Tensor:
+        """q, k: [T, H, Dk]; v: [T, H, Dv] as projected; returns [T, H * Dv] float32."""
+        ctx = get_context()
+        return ops.fixed_decay_memory(q, k, v, self.decay, cache["state"], ctx.cu_seqlens_q, ctx.cu_seqlens_k, ctx.state_slots,
+                                      ctx.max_seqlen_q, ctx.min_seqlen_q)

@@ -6,7 +6,9 @@ sequence carried in ``state[slot]``.  ``DecayMemory``: S <- diag(w) S + k v^T wi
 and key channel, read BEFORE the write as (S + diag(bonus) k v^T)^T r, normalised per head and gated by SiLU.
 ``ConvBiasSilu``: a short causal convolution with bias, then SiLU.  ``StateSpaceScan``: S <- a S + dt B x^T with one
 scalar decay a = exp(-exp(A_log) dt) per head and step, dt = softplus(dt_raw + dt_bias), read AFTER the write as
-S^T C + D x, times silu(z), in float32; ``group_rms_norm`` follows it.
+S^T C + D x, times silu(z), in float32; ``group_rms_norm`` follows it.  ``SelectiveScan``: one diagonal recurrence per CHANNEL,
+S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n with a step size dt = softplus(dt_raw + dt_bias) per token and channel and
+A = -exp(A_log), read after the write as sum_n S[c, n] C_n + D_c x_c, times silu(z); its state is [channels, states].
 
 The states [H, Dk, Dv] live in float32 in ``state[slot]``.  A slot is a row of the state tensors; the step's
 ``CacheContext.state_slots`` names the slot of every sequence of the batch.  A sequence whose rows start at position 0
@@ -80,3 +82,28 @@ class StateSpaceScan(nn.Module):
         ctx = get_context()
         return ops.state_space_scan(x, B, C, dt_raw, z, self.dt_bias, self.A_log, self.D, state, ctx.cu_seqlens_q,
                                     ctx.cu_seqlens_k, ctx.state_slots)
+
+
+class SelectiveScan(nn.Module):
+    def __init__(self, channels: int, states: int, device=None):
+        super().__init__()
+        self.channels, self.states = channels, states
+        f32 = dict(dtype=torch.float32, device=device)
+        self.dt_bias = nn.Parameter(torch.zeros(channels, **f32))
+        self.A_log = nn.Parameter(torch.zeros(channels, states, **f32))
+        self.D = nn.Parameter(torch.zeros(channels, **f32))
+        self.register_buffer("A", torch.full((channels, states), -1.0, **f32), persistent=False)
+
+    def finalize(self) -> None:
+        """After loading: the rates as the scan takes them."""
+        self.A = (-torch.exp(self.A_log.data)).contiguous()
+
+    def state_shapes(self) -> dict:
+        return {"state": ((self.channels, self.states), torch.float32)}
+
+    def forward(self, x, dt_raw, z, B, C, state: torch.Tensor) -> torch.Tensor:
+        """x, dt_raw, z: [T, channels]; B, C: [T, states]; state [slots, channels, states] float32.  Returns y * silu(z) in
+        x's dtype, [T, channels]."""
+        ctx = get_context()
+        return ops.selective_scan(x, dt_raw, z, B, C, self.dt_bias, self.A, self.D, state, ctx.cu_seqlens_q, ctx.cu_seqlens_k,
+                                  ctx.state_slots, ctx.max_seqlen_q)

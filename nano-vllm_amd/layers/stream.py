@@ -6,7 +6,7 @@ times a multiplier, an RMS-normed side input is added times the same multiplier,
 dtype, and / or the next layer's grouped RMS norm is taken (the row is cut into equal consecutive parts, each divided by
 its own root mean square).  ``CausalConvAdd``: x + a short causal convolution of x over time per channel, the last taps-1
 inputs of each sequence carried in float32 in ``state[slot]``.  ``TokenGate``: gelu_tanh(z) times a slice of a per-token
-table row.  The modules own no state: a layer that runs several times per forward has one state per run, passed in.
+table row.  ``ScaledNorm``: the weight of an RMS norm whose output is also scaled per column, as the boundary takes it.  The modules own no state: a layer that runs several times per forward has one state per run, passed in.
 """
 from __future__ import annotations
 
@@ -41,3 +41,17 @@ class TokenGate(nn.Module):
 
     def forward(self, z: torch.Tensor, table: torch.Tensor, ids: torch.Tensor) -> torch.Tensor:
         return ops.token_gate(z, table, ids, self.offset, self.dim)
+
+
+class ScaledNorm(nn.Module):
+    """Norm weight w and column scale s of a sublayer's output; `applied` is w * s in float32 (refreshed by `finalize()` after
+    loading), what ``stream_boundary`` multiplies the normed input by."""
+
+    def __init__(self, width: int, device=None):
+        super().__init__()
+        self.weight = nn.Parameter(torch.ones(width, dtype=torch.float32, device=device))
+        self.scale = nn.Parameter(torch.ones(width, dtype=torch.float32, device=device))
+        self.register_buffer("applied", torch.ones(width, dtype=torch.float32, device=device), persistent=False)
+
+    def finalize(self) -> None:
+        self.applied = (self.weight.data.float() * self.scale.data.float()).contiguous()

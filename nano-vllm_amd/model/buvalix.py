@@ -146,11 +146,17 @@ def _linear(n_in, n_out, bias, dtype, device):
 
 class _FusedInputs:
     """Several projections of one input run as ONE matrix product: after `fuse()` the named nn.Linear weights are
-    views of one [sum of outputs, inputs] tensor (names and values unchanged)."""
+    views of one [sum of outputs, inputs] tensor (names and values unchanged).  `multiple`: zero rows are added so that the
+    product's rows are a multiple of that many elements apart (aligned for vector access)."""
 
-    def _fuse(self, names):
+    def _fuse(self, names, multiple: int = 1):
         mods = [getattr(self, n) for n in names]
-        w = torch.cat([m.weight.data for m in mods], dim=0)
+        rows = [m.weight.data for m in mods]
+        pad = -sum(r.shape[0] for r in rows) % multiple
+        if pad:
+            assert mods[0].bias is None
+            rows.append(rows[0].new_zeros(pad, rows[0].shape[1]))
+        w = torch.cat(rows, dim=0)
         has_bias = mods[0].bias is not None
         b = torch.cat([m.bias.data for m in mods], dim=0) if has_bias else None
         o = 0
@@ -161,12 +167,12 @@ class _FusedInputs:
                 m.bias.data = b[o:o + n]
             o += n
         self._fused_w, self._fused_b = w, b
-        self._fused_sizes = [m.weight.shape[0] for m in mods]
+        self._fused_sizes = [m.weight.shape[0] for m in mods] + ([pad] if pad else [])
 
     def _project(self, x, names):
         w = getattr(self, "_fused_w", None)
         if w is not None and w.device == x.device and w.dtype == x.dtype:
-            return F.linear(x, w, self._fused_b).split(self._fused_sizes, dim=1)
+            return F.linear(x, w, self._fused_b).split(self._fused_sizes, dim=1)[:len(names)]
         return tuple(getattr(self, n)(x) for n in names)
 
 

@@ -129,6 +129,16 @@ def _nekodra_model(cfg, dtype=torch.bfloat16, device="cuda", **kw):
     return NekodraForCausalLM(cfg, dtype=dtype, device=device, **kw)
 
 
+def _tiralix_config(raw: dict):
+    from .tiralix import TiralixConfig
+    return TiralixConfig.from_dict(raw)
+
+
+def _tiralix_model(cfg, dtype=torch.bfloat16, device="cuda", **kw):
+    from .tiralix import TiralixForCausalLM
+    return TiralixForCausalLM(cfg, dtype=dtype, device=device, **kw)
+
+
 register(["Qwen3ForCausalLM", "Qwen3"], _qwen3_config, lambda cfg, **kw: _qwen3_model(cfg, **kw))
 register(["LlamaForCausalLM", "Llama"], lambda raw: _qwen3_config({**raw, "qk_norm": False}),
          lambda cfg, **kw: _qwen3_model(cfg, **kw))
@@ -137,3 +147,4 @@ register(["Benarax", "BenaraxForCausalLM"], _benarax_config, _benarax_model)
 register(["Divadra", "DivadraForCausalLM"], _divadra_config, _divadra_model)
 register(["Tutedra", "TutedraForCausalLM"], _tutedra_config, _tutedra_model)
 register(["Nekodra", "NekodraForCausalLM"], _nekodra_config, _nekodra_model)
+register(["Tiralix", "TiralixForCausalLM"], _tiralix_config, _tiralix_model)

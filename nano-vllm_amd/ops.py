@@ -1545,3 +1545,148 @@ def moe_route_softmax(logits: torch.Tensor, correction: Optional[torch.Tensor], 
                                   int(top), float(scale), _stream(logits))
     _lib.check(rc, "nv_moe_route_softmax", dll)
     return ids, wgt
+
+
+# ---------------------------------------------------------------------------------------------------------
+# Two mixers side by side on one input (softmax attention with whole-row norms and head gates; a linear memory with a fixed
+# decay), a selective scan, a clamped gated unit, scaled and soft-capped logits.
+# ---------------------------------------------------------------------------------------------------------
+def selective_scan(x: torch.Tensor, dt_raw: torch.Tensor, z: torch.Tensor, Bm: torch.Tensor, Cm: torch.Tensor,
+                   dt_bias: torch.Tensor, A: torch.Tensor, D_skip: torch.Tensor, state: torch.Tensor, cu_seqlens_q: torch.Tensor,
+                   cu_seqlens_k: torch.Tensor, state_slots: torch.Tensor, max_seqlen_q: int) -> torch.Tensor:
+    """Diagonal recurrence per channel with token-dependent decay and input over a step's rows; state [slots, C, N] float32
+    updated in place; x, dt_raw, z: [T, C]; Bm, Cm: [T, N]; A [C, N] float32 (negative); returns y * silu(z), [T, C]."""
+    dt = _dt(x, "x")
+    T, Cc = x.shape
+    N = Bm.shape[1]
+    for t, n, cols in ((x, "x", Cc), (dt_raw, "dt_raw", Cc), (z, "z", Cc), (Bm, "B", N), (Cm, "C", N)):
+        _rows2d(t, n)
+        _need(t.is_cuda and t.shape == (T, cols) and t.dtype == x.dtype, f"{n} must be [T, {cols}] of x's dtype")
+    _need(state.is_cuda and state.dtype == torch.float32 and state.is_contiguous() and state.shape[1:] == (Cc, N),
+          "state must be contiguous float32 [slots, channels, states]")
+    _need(dt_bias.numel() == Cc and A.shape == (Cc, N) and D_skip.numel() == Cc, "constant shapes")
+    B = _seq_meta(cu_seqlens_q, cu_seqlens_k, state_slots)
+    out = torch.empty((T, Cc), dtype=x.dtype, device=x.device)
+    if T == 0:
+        return out
+    dll = _lib.mixers()
+    mq = max(int(max_seqlen_q), 1)
+    need = dll.nv_selective_scan_workspace_bytes(B, Cc, N, mq)
+    ws = _workspace(x.device, need) if need else None
+    rc = dll.nv_selective_scan(x.data_ptr(), x.stride(0), dt_raw.data_ptr(), dt_raw.stride(0), z.data_ptr(), z.stride(0),
+                               Bm.data_ptr(), Bm.stride(0), Cm.data_ptr(), Cm.stride(0), _f32c(dt_bias, "dt_bias"),
+                               _f32c(A, "A"), _f32c(D_skip, "D"), state.data_ptr(), out.data_ptr(), out.stride(0),
+                               cu_seqlens_q.data_ptr(), cu_seqlens_k.data_ptr(), state_slots.data_ptr(), B, Cc, N, mq, dt,
+                               _ptr(ws), ws.numel() if ws is not None else 0, _stream(x))
+    _lib.check(rc, "nv_selective_scan", dll)
+    return out
+
+
+def fixed_decay_memory(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor, state: torch.Tensor,
+                       cu_seqlens_q: torch.Tensor, cu_seqlens_k: torch.Tensor, state_slots: torch.Tensor, max_seqlen_q: int,
+                       min_seqlen_q: int = 0) -> torch.Tensor:
+    """S <- decay_h S + silu(k) silu(v)^T, o = S^T silu(q) over a step's rows; q, k: [T, H, Dk]; v: [T, H, Dv] as projected;
+    decay [H] float32; state [slots, H, Dk, Dv] float32 updated in place; returns o as float32 [T, H * Dv]."""
+    dt = _dt(q, "q")
+    T, H, Dk = q.shape
+    Dv = v.shape[2]
+    for t, n in ((q, "q"), (k, "k"), (v, "v")):
+        _rows_ok(t, n)
+        _need(t.dtype == q.dtype, "q, k, v must have one dtype")
+    _need(k.shape == (T, H, Dk) and v.shape[:2] == (T, H) and decay.numel() == H, "q / k / v / decay shapes differ")
+    _need(state.is_cuda and state.dtype == torch.float32 and state.is_contiguous() and state.shape[1:] == (H, Dk, Dv),
+          "state must be contiguous float32 [slots, H, Dk, Dv]")
+    B = _seq_meta(cu_seqlens_q, cu_seqlens_k, state_slots)
+    out = torch.empty((T, H * Dv), dtype=torch.float32, device=q.device)
+    if T == 0:
+        return out
+    dll = _lib.mixers()
+    mq = max(int(max_seqlen_q), 1)
+    need = dll.nv_fixed_decay_workspace_bytes(B, H, Dk, Dv, mq, dt)
+    ws = _workspace(q.device, need) if need else None
+    rc = dll.nv_fixed_decay_memory(q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0), k.stride(0), v.stride(0),
+                                   _f32c(decay, "decay"), state.data_ptr(), out.data_ptr(), out.stride(0),
+                                   cu_seqlens_q.data_ptr(), cu_seqlens_k.data_ptr(), state_slots.data_ptr(), B, H, Dk, Dv, mq,
+                                   int(min_seqlen_q), dt, _ptr(ws), ws.numel() if ws is not None else 0, _stream(q))
+    _lib.check(rc, "nv_fixed_decay_memory", dll)
+    return out
+
+
+def row_norm_rope_store(positions: torch.Tensor, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, q_norm: torch.Tensor,
+                        k_norm: torch.Tensor, eps: float, freq: Optional[torch.Tensor], rot_dims: int, magnitude: float,
+                        slot_mapping: Optional[torch.Tensor], k_cache: torch.Tensor, v_cache: torch.Tensor) -> torch.Tensor:
+    """RMS norm over the whole q [T, H, D] / k [T, G, D] rows (weights [H * D], [G * D]), rotate-half rotary on the first
+    rot_dims dimensions of every head (cos and sin times magnitude), scatter of k and v [T, G, Dv] into the paged cache;
+    returns the prepared q."""
+    dt = _dt(q, "q")
+    for t, n in ((q, "q"), (k, "k"), (v, "v")):
+        _rows_ok(t, n)
+        _need(t.dtype == q.dtype, "q, k, v must have one dtype")
+    T, H, D = q.shape
+    G, Dv = k.shape[1], v.shape[2]
+    _need(k.shape == (T, G, D) and v.shape[:2] == (T, G), "k / v rows do not match q")
+    _need(q_norm.numel() == H * D and k_norm.numel() == G * D, "the norm weights span the whole q / k rows")
+    _need(positions.is_cuda and positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() == T,
+          "positions must be a contiguous int64 [tokens] GPU tensor")
+    if rot_dims:
+        _need(freq is not None and freq.numel() == rot_dims // 2, "freq must hold rot_dims / 2 frequencies")
+    if slot_mapping is not None:
+        _i32(slot_mapping, "slot_mapping")
+        _need(slot_mapping.numel() == T, "slot_mapping length != number of tokens")
+    _need(k_cache.is_cuda and v_cache.is_cuda and k_cache.is_contiguous() and v_cache.is_contiguous() and k_cache.dtype == q.dtype
+          and v_cache.dtype == q.dtype and k_cache.dim() == 4 and k_cache.shape[2:] == (G, D) and v_cache.shape[2:] == (G, Dv)
+          and k_cache.shape[:2] == v_cache.shape[:2], "caches must be contiguous [num_blocks, block_size, G, D] and [.., G, Dv] of q's dtype")
+    q_out = torch.empty((T, H, D), dtype=q.dtype, device=q.device)
+    dll = _lib.mixers()
+    rc = dll.nv_row_norm_rope_store(q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0), k.stride(0), v.stride(0),
+                                    _f32c(q_norm, "q_norm"), _f32c(k_norm, "k_norm"), float(eps), _f32c(freq, "freq") or None,
+                                    int(rot_dims), float(magnitude), positions.data_ptr(), _ptr(slot_mapping), q_out.data_ptr(),
+                                    k_cache.data_ptr(), v_cache.data_ptr(), dt, T, H, G, D, Dv, _stream(q))
+    _lib.check(rc, "nv_row_norm_rope_store", dll)
+    return q_out
+
+
+def join_gated(attn: torch.Tensor, head_gate: torch.Tensor, left_scale: float, mem: torch.Tensor, norm_weight: torch.Tensor,
+               gate: torch.Tensor, eps: float, right_scale: float) -> torch.Tensor:
+    """[left_scale * sigmoid(head_gate) * attn | right_scale * sigmoid(gate) * rmsnorm(mem) * norm_weight] as the rows of one
+    output product; attn [T, H * Dv], head_gate [T, H], gate [T, cols] of one dtype, mem [T, cols] float32."""
+    dt = _dt(attn, "attn")
+    T, cols = mem.shape
+    H = head_gate.shape[1]
+    for t, n in ((attn, "attn"), (head_gate, "head_gate"), (gate, "gate"), (mem, "mem")):
+        _rows2d(t, n)
+        _need(t.is_cuda and t.shape[0] == T, f"{n} rows differ")
+    _need(head_gate.dtype == attn.dtype and gate.dtype == attn.dtype and mem.dtype == torch.float32, "dtypes")
+    _need(attn.shape[1] % H == 0 and gate.shape[1] == cols and norm_weight.numel() == cols, "column counts differ")
+    y = torch.empty((T, attn.shape[1] + cols), dtype=attn.dtype, device=attn.device)
+    dll = _lib.mixers()
+    rc = dll.nv_join_gated(attn.data_ptr(), attn.stride(0), head_gate.data_ptr(), head_gate.stride(0), H, attn.shape[1] // H,
+                           float(left_scale), mem.data_ptr(), mem.stride(0), _f32c(norm_weight, "norm_weight"), gate.data_ptr(),
+                           gate.stride(0), cols, float(eps), float(right_scale), y.data_ptr(), dt, T, _stream(attn))
+    _lib.check(rc, "nv_join_gated", dll)
+    return y
+
+
+def clamped_glu_rows(x: torch.Tensor, limit: float, alpha: float, shift: float) -> torch.Tensor:
+    """g sigmoid(alpha g) (u + shift) with g = min(gate, limit), u = clamp(up, -limit, limit) for x = [gate | up]."""
+    _rows2d(x, "x")
+    dt = _dt(x, "x")
+    inter = x.shape[1] // 2
+    _need(x.shape[1] == 2 * inter, "x must hold [gate | up]")
+    y = torch.empty((x.shape[0], inter), dtype=x.dtype, device=x.device)
+    dll = _lib.mixers()
+    rc = dll.nv_clamped_glu_rows(x.data_ptr(), x.stride(0), y.data_ptr(), dt, x.shape[0], inter, float(limit), float(alpha),
+                                 float(shift), _stream(x))
+    _lib.check(rc, "nv_clamped_glu_rows", dll)
+    return y
+
+
+def scale_softcap(x: torch.Tensor, scale: float, cap: float) -> torch.Tensor:
+    """cap * tanh(scale * x / cap) in float32 (cap 0: scale * x)."""
+    dt = _dt(x, "x")
+    _need(x.is_contiguous(), "x must be contiguous")
+    y = torch.empty(x.shape, dtype=torch.float32, device=x.device)
+    dll = _lib.mixers()
+    _lib.check(dll.nv_scale_softcap(x.data_ptr(), y.data_ptr(), dt, x.numel(), float(scale), float(cap), _stream(x)),
+               "nv_scale_softcap", dll)
+    return y
