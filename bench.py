@@ -77,6 +77,9 @@ def parse():
     ap.add_argument("--nekodra", action="store_true",
                     help="instead of the default workload: the Nekodra kernels and model beside Benarax at equal sizes "
                          "(one GPU, random weights), one JSON line")
+    ap.add_argument("--tiralix", action="store_true",
+                    help="instead of the default workload: the Tiralix kernels and model beside Tutedra and Buvalix at equal "
+                         "sizes (one GPU, random weights), one JSON line")
     return ap.parse_args()
 
 
@@ -820,6 +823,12 @@ def main():
             raise SystemExit("bench.py needs a GPU (the hot path has no CPU implementation)")
         from tools.nekodra_bench import run as nekodra_run
         print(json.dumps(nekodra_run("cuda:0")))
+        return
+    if args.tiralix:
+        if not torch.cuda.is_available():
+            raise SystemExit("bench.py needs a GPU (the hot path has no CPU implementation)")
+        from tools.tiralix_bench import run as tiralix_run
+        print(json.dumps(tiralix_run("cuda:0")))
         return
     if args.divadra:
         if not torch.cuda.is_available():
