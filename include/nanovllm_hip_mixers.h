@@ -474,15 +474,21 @@ NV_API int nv_selective_scan(const void* x, int64_t x_stride, const void* dt_raw
 /*
  * Linear attention with one constant decay per head, state [num_slots, H, Dk, Dv] fp32 carried per sequence:
  *   S <- decay_h S + silu(k) silu(v)^T;  o = S^T silu(q)              (out: [T, H * Dv] fp32 with a row stride)
- * q, k: [T, H * Dk]; v: [T, H * Dv] of dtype with row strides; decay: [H] fp32.  Dk, Dv <= 256.  max_seqlen_q / min_seqlen_q:
- * the most and fewest rows a sequence has in the step (min_seqlen_q 0: not known); long portions of bf16 rows with Dk <= 128
- * run in chunks on the matrix cores, through a workspace when a step with few sequences is cut into segments along time.
+ * q, k: [T, H * Dk]; v: [T, H * Dv] of dtype with row strides; decay: [H] fp32.  Dk, Dv <= 256.  max_seqlen_q: the most rows
+ * a sequence has in the step; `portions`: which kinds of portions the step may hold, NV_PORTION_* added up (7: anything; a
+ * kind left out is not run).  Single tokens stream the state, portions of at most NV_FEW_ROWS tokens run token by token, longer
+ * ones of bf16 rows with Dk <= 128 in chunks on the matrix cores, through a workspace when a step with few sequences is cut
+ * into segments along time.
  */
+#define NV_FEW_ROWS 16
+#define NV_PORTION_SINGLE 1
+#define NV_PORTION_FEW 2
+#define NV_PORTION_LONG 4
 NV_API int64_t nv_fixed_decay_workspace_bytes(int num_seqs, int H, int Dk, int Dv, int max_seqlen_q, int dtype);
 NV_API int nv_fixed_decay_memory(const void* q, const void* k, const void* v, int64_t q_stride, int64_t k_stride,
                                  int64_t v_stride, const float* decay, float* state, float* out, int64_t out_stride,
                                  const int32_t* cu_seqlens_q, const int32_t* cu_seqlens_k, const int32_t* state_slots,
-                                 int num_seqs, int H, int Dk, int Dv, int max_seqlen_q, int min_seqlen_q, int dtype,
+                                 int num_seqs, int H, int Dk, int Dv, int max_seqlen_q, int portions, int dtype,
                                  void* workspace, int64_t workspace_bytes, void* stream);
 
 /*

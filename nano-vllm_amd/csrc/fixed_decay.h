@@ -16,7 +16,8 @@ struct FixedDecayArgs {
     int num_seqs, H, Dk, Dv;
 };
 
-// Token by token, every sequence with at most max_rows rows in the step (0: every sequence); any sizes up to 256 x 256.
-int launch_fixed_decay_rows(const FixedDecayArgs& f, int dtype, int max_rows, hipStream_t s);
+// Token by token with the state in registers, every sequence with min_rows .. max_rows rows in the step; any sizes up to
+// 256 x 256.
+int launch_fixed_decay_rows(const FixedDecayArgs& f, int dtype, int min_rows, int max_rows, hipStream_t s);
 
 }  // namespace nv

@@ -2,7 +2,8 @@
 //
 //   q = silu(q_raw), k = silu(k_raw), v = silu(v_raw);   S_t = decay_h S_(t-1) + k_t v_t^T;   o_t = S_t^T q_t
 //
-// Portions of a few tokens run token by token (gated_memory.hip); longer ones in chunks of 64 tokens on the matrix cores:
+// Single tokens stream the state through once (read, decayed, written, read out); portions of a few tokens run token by token
+// with the state in registers (gated_memory.hip); longer ones in chunks of 64 tokens on the matrix cores:
 // with tokens i, j of a chunk and the state S in front of it
 //
 //   o_i = decay^(i+1) S^T q_i + sum_(j <= i) decay^(i-j) (q_i . k_j) v_j
@@ -25,6 +26,7 @@
 
 #include "fixed_decay.h"
 #include "mfma_tile.h"
+#include "row_pieces.h"
 #include "../../include/nanovllm_hip_mixers.h"
 
 namespace nv {
@@ -32,7 +34,7 @@ namespace nv {
 typedef __attribute__((address_space(3))) s16x4 fd_lds_s16x4;
 
 constexpr int kFdChunk = 64;
-constexpr int kFdFewRows = 16;                 // portions of at most this many tokens run token by token
+constexpr int kFdFewRows = NV_FEW_ROWS;                 // portions of at most this many tokens run token by token
 constexpr int kFdVs = 64 + 8;                  // LDS row of the values, in elements
 
 struct FdParams {
@@ -289,6 +291,82 @@ __global__ __launch_bounds__(256) void fixed_decay_chunk_kernel(const FdParams p
     }
 }
 
+// ------------------------------------------------------------------------------------------------ one token
+// One workgroup per (sequence, head): V value columns per thread (16-byte pieces of the state's rows), the rows over the
+// thread groups, eight rows of a thread in flight; the groups' parts of o meet in LDS.
+template <typename T, int V>
+__global__ __launch_bounds__(256) void fixed_decay_single_kernel(const FixedDecayArgs f, int pieces) {
+    constexpr int U = 8;
+    extern __shared__ __attribute__((aligned(16))) float fd_smem[];
+    const int H = f.H, Dk = f.Dk, Dv = f.Dv;
+    float *ks = fd_smem, *qs = ks + Dk, *os = qs + Dk;           // [Dk], [Dk], [groups][Dv]
+    const int b = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
+    const int t = f.cu_q[b];
+    if (f.cu_q[b + 1] - t != 1) return;
+    const bool fresh = f.cu_k[b + 1] - f.cu_k[b] == 1;
+    for (int d = tid; d < Dk; d += 256) {
+        const float k = (float)((const T*)f.k)[(int64_t)t * f.k_stride + (int64_t)h * Dk + d];
+        const float q = (float)((const T*)f.q)[(int64_t)t * f.q_stride + (int64_t)h * Dk + d];
+        ks[d] = k / (1.0f + expf(-k));
+        qs[d] = q / (1.0f + expf(-q));
+    }
+    const int c = (tid % pieces) * V, group = tid / pieces, groups = 256 / pieces;      // (pieces is a power of two)
+    const bool live = c < Dv;
+    float v[V], o[V];
+#pragma unroll
+    for (int e = 0; e < V; ++e) {
+        v[e] = live ? (float)((const T*)f.v)[(int64_t)t * f.v_stride + (int64_t)h * Dv + c + e] : 0.f;
+        v[e] = v[e] / (1.0f + expf(-v[e]));
+        o[e] = 0.f;
+    }
+    const float decay = f.decay[h];
+    float* st = f.state + ((int64_t)f.slots[b] * H + h) * (int64_t)Dk * Dv + c;
+    __syncthreads();
+    for (int d0 = group; d0 < Dk; d0 += groups * U) {
+        Cols<V> s[U];
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            const int d = d0 + u * groups;
+#pragma unroll
+            for (int e = 0; e < V; ++e) s[u].v[e] = 0.f;
+            if (live && d < Dk && !fresh) s[u] = row_load<V>(st + (int64_t)d * Dv);
+        }
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            const int d = d0 + u * groups;
+            if (d >= Dk) break;
+#pragma unroll
+            for (int e = 0; e < V; ++e) {
+                s[u].v[e] = decay * s[u].v[e] + ks[d] * v[e];
+                o[e] += s[u].v[e] * qs[d];
+            }
+            if (live) row_store<V>(st + (int64_t)d * Dv, s[u]);
+        }
+    }
+    if (live) {
+#pragma unroll
+        for (int e = 0; e < V; ++e) os[group * Dv + c + e] = o[e];
+    }
+    __syncthreads();
+    for (int i = tid; i < Dv; i += 256) {
+        float sum = 0.f;
+        for (int j = 0; j < groups; ++j) sum += os[j * Dv + i];
+        f.out[(int64_t)t * f.out_stride + (int64_t)h * Dv + i] = sum;
+    }
+}
+
+template <typename T>
+static void launch_single(const FixedDecayArgs& f, hipStream_t s) {
+    const bool vec = f.Dv % 4 == 0;                              // (states start on 16 bytes, slots are whole rows)
+    const int cols = vec ? f.Dv / 4 : f.Dv;
+    int pieces = 1;
+    while (pieces < cols) pieces *= 2;                           // at most 256
+    const size_t lds = sizeof(float) * (2 * (size_t)f.Dk + (size_t)(256 / pieces) * f.Dv);
+    const dim3 grid((unsigned)f.num_seqs, (unsigned)f.H), block(256);
+    if (vec) hipLaunchKernelGGL((fixed_decay_single_kernel<T, 4>), grid, block, lds, s, f, pieces);
+    else hipLaunchKernelGGL((fixed_decay_single_kernel<T, 1>), grid, block, lds, s, f, pieces);
+}
+
 struct FdPlan {
     int nseg, seg_len;
     int64_t ws_floats;
@@ -336,10 +414,10 @@ extern "C" int64_t nv_fixed_decay_workspace_bytes(int num_seqs, int H, int Dk, i
 extern "C" int nv_fixed_decay_memory(const void* q, const void* k, const void* v, int64_t q_stride, int64_t k_stride,
                                      int64_t v_stride, const float* decay, float* state, float* out, int64_t out_stride,
                                      const int32_t* cu_seqlens_q, const int32_t* cu_seqlens_k, const int32_t* state_slots,
-                                     int num_seqs, int H, int Dk, int Dv, int max_seqlen_q, int min_seqlen_q, int dtype,
+                                     int num_seqs, int H, int Dk, int Dv, int max_seqlen_q, int portions, int dtype,
                                      void* workspace, int64_t workspace_bytes, void* stream) {
     using namespace nv;
-    NV_REQUIRE(num_seqs >= 0 && H > 0 && Dk > 0 && Dv > 0 && max_seqlen_q >= 1 && min_seqlen_q >= 0, NV_ERR_INVALID_ARG,
+    NV_REQUIRE(num_seqs >= 0 && H > 0 && Dk > 0 && Dv > 0 && max_seqlen_q >= 1, NV_ERR_INVALID_ARG,
                "nv_fixed_decay_memory: bad sizes");
     if (num_seqs == 0) return NV_OK;
     NV_REQUIRE(q && k && v && decay && state && out && cu_seqlens_q && cu_seqlens_k && state_slots, NV_ERR_INVALID_ARG,
@@ -351,16 +429,24 @@ extern "C" int nv_fixed_decay_memory(const void* q, const void* k, const void* v
     FdParams p{};
     p.f = FixedDecayArgs{q,          k,          v,          q_stride, k_stride, v_stride, decay, state, out,
                          out_stride, cu_seqlens_q, cu_seqlens_k, state_slots, num_seqs, H,        Dk,       Dv};
+    // the launches a sequence of this many rows belongs to
     const bool chunked = fd_chunked(Dk, Dv, dtype, max_seqlen_q);
-    if (!chunked) return launch_fixed_decay_rows(p.f, dtype, 0, s);
+    if (portions & NV_PORTION_SINGLE) {
+        NV_REQUIRE((uintptr_t)state % 16 == 0, NV_ERR_INVALID_ARG, "nv_fixed_decay_memory: the state must start on 16 bytes");
+        if (dtype == NV_DTYPE_BF16) launch_single<__bf16>(p.f, s);
+        else launch_single<float>(p.f, s);
+        const int rc = check_launch("nv_fixed_decay_memory (single tokens)");
+        if (rc != NV_OK) return rc;
+    }
+    if ((portions & NV_PORTION_FEW) || (!chunked && (portions & NV_PORTION_LONG))) {
+        const int rc = launch_fixed_decay_rows(p.f, dtype, 2, chunked ? kFdFewRows : 1 << 30, s);
+        if (rc != NV_OK) return rc;
+    }
+    if (!chunked || !(portions & NV_PORTION_LONG)) return NV_OK;
     const FdPlan plan = fd_plan(num_seqs, H, Dk, Dv, max_seqlen_q);
     NV_REQUIRE(plan.ws_floats == 0 || (workspace && workspace_bytes >= plan.ws_floats * (int64_t)sizeof(float)), NV_ERR_WORKSPACE,
                "nv_fixed_decay_memory: workspace of %lld bytes, need %lld", (long long)workspace_bytes,
                (long long)(plan.ws_floats * (int64_t)sizeof(float)));
-    if (min_seqlen_q <= kFdFewRows) {
-        const int rc = launch_fixed_decay_rows(p.f, dtype, kFdFewRows, s);
-        if (rc != NV_OK) return rc;
-    }
     p.nseg = plan.nseg;
     p.seg_len = plan.seg_len;
     p.seg_state = (float*)workspace;

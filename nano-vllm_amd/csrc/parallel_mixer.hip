@@ -192,7 +192,10 @@ __global__ __launch_bounds__(256) void clamped_glu_rows_kernel(const T* __restri
 #pragma unroll
     for (int e = 0; e < V; ++e) {
         const float gg = fminf(g.v[e], limit), uu = fminf(fmaxf(u.v[e], -limit), limit);
-        o.v[e] = gg / (1.0f + expf(-alpha * gg)) * (uu + shift);
+        if constexpr (sizeof(T) == 2)      // (the result is rounded to bf16: the hardware's exponential and reciprocal are enough)
+            o.v[e] = gg * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * alpha * gg)) * (uu + shift);
+        else
+            o.v[e] = gg / (1.0f + expf(-alpha * gg)) * (uu + shift);
     }
     row_store<V>(y + r * inter + c, o);
 }
@@ -294,17 +297,17 @@ extern "C" int nv_clamped_glu_rows(const void* x, int64_t x_stride, void* y, int
     NV_REQUIRE(x && y, NV_ERR_INVALID_ARG, "nv_clamped_glu_rows: null pointer");
     NV_REQUIRE(dtype == NV_DTYPE_BF16 || dtype == NV_DTYPE_F32, NV_ERR_INVALID_ARG, "nv_clamped_glu_rows: bad dtype");
     const bool bf = dtype == NV_DTYPE_BF16;
-    const bool vec = inter % 4 == 0 && x_stride % 4 == 0 && ((uintptr_t)x | (uintptr_t)y) % (bf ? 8 : 16) == 0;
-    const int pieces = vec ? inter / 4 : inter;
+    const bool vec = inter % 8 == 0 && x_stride % 8 == 0 && ((uintptr_t)x | (uintptr_t)y) % 16 == 0;
+    const int pieces = vec ? inter / 8 : inter;
     const int64_t n = rows * pieces, grid = (n + 255) / 256;
     NV_REQUIRE(grid < (1LL << 31), NV_ERR_UNSUPPORTED, "nv_clamped_glu_rows: launch too large");
     hipStream_t s = (hipStream_t)stream;
 #define NV_GLU(T, V)                                                                                                 \
     hipLaunchKernelGGL((clamped_glu_rows_kernel<T, V>), dim3((unsigned)grid), dim3(256), 0, s, (const T*)x, x_stride, \
                        (T*)y, inter, pieces, n, limit, alpha, shift)
-    if (bf && vec) NV_GLU(__bf16, 4);
+    if (bf && vec) NV_GLU(__bf16, 8);
     else if (bf) NV_GLU(__bf16, 1);
-    else if (vec) NV_GLU(float, 4);
+    else if (vec) NV_GLU(float, 8);
     else NV_GLU(float, 1);
 #undef NV_GLU
     return check_launch("nv_clamped_glu_rows");

@@ -27,8 +27,49 @@ namespace nv {
 constexpr int kScThreads = 256;
 constexpr int kScTile = 16;                    // tokens prepared at a time
 
-__device__ __forceinline__ float sc_softplus(float x) { return x > 20.f ? x : log1pf(expf(x)); }
-__device__ __forceinline__ float sc_silu(float x) { return x / (1.0f + expf(-x)); }
+constexpr float kScLog2e = 1.4426950408889634f, kScLn2 = 0.6931471805599453f;
+
+// log(1 + exp(x)) = max(x, 0) + log1p(u), u = exp(-|x|); log1p(u) = u log(w) / (w - 1) with w = 1 + u rounded (the rounding
+// of w cancels: D. Goldberg, "What Every Computer Scientist Should Know About Floating-Point Arithmetic", theorem 4).
+__device__ __forceinline__ float sc_softplus(float x) {
+    const float u = __builtin_amdgcn_exp2f(-fabsf(x) * kScLog2e), w = 1.0f + u, d = w - 1.0f;
+    const float l = d == 0.f ? u : __builtin_amdgcn_logf(w) * kScLn2 * (u * __builtin_amdgcn_rcpf(d));
+    return fmaxf(x, 0.f) + l;
+}
+__device__ __forceinline__ float sc_silu(float x) {
+    return x * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-kScLog2e * x));
+}
+
+// The SPL states n0 .. of a channel's row of N: in pieces of four where the row allows it.  `in` says whether the lane has any.
+template <int SPL>
+__device__ __forceinline__ void sc_load_states(const float* row, int n0, int N, bool in, float* s) {
+#pragma unroll
+    for (int i = 0; i < SPL; i += 4) {
+        float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (N % 4 == 0) {
+            if (in && n0 + i < N) v = *(const float4*)(row + n0 + i);
+        } else if (in) {
+            if (n0 + i < N) v.x = row[n0 + i];
+            if (n0 + i + 1 < N) v.y = row[n0 + i + 1];
+            if (n0 + i + 2 < N) v.z = row[n0 + i + 2];
+            if (n0 + i + 3 < N) v.w = row[n0 + i + 3];
+        }
+        s[i] = v.x; s[i + 1] = v.y; s[i + 2] = v.z; s[i + 3] = v.w;
+    }
+}
+template <int SPL>
+__device__ __forceinline__ void sc_store_states(float* row, int n0, int N, const float* s) {
+#pragma unroll
+    for (int i = 0; i < SPL; i += 4) {
+        if (N % 4 == 0) {
+            if (n0 + i < N) *(float4*)(row + n0 + i) = make_float4(s[i], s[i + 1], s[i + 2], s[i + 3]);
+        } else {
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+                if (n0 + i + e < N) row[n0 + i + e] = s[i + e];
+        }
+    }
+}
 
 // Sum over aligned groups of L lanes; every lane of the group gets it.
 template <int L>
@@ -89,49 +130,35 @@ __global__ __launch_bounds__(kScThreads) void selective_scan_kernel(const ScArgs
     const int C = a.C, N = a.N, c = c0 + ch;
     const bool live = c < C;
     float* slot_state = a.state + ((int64_t)a.slots[b] * C + c) * N;
+    const int n0 = sub * SPL;
     float A2[SPL], S[SPL];                                       // A log2(e); the state
+    sc_load_states<SPL>(a.A + (int64_t)c * N, n0, N, live, A2);
 #pragma unroll
     for (int i = 0; i < SPL; ++i) {
-        const int n = sub * SPL + i;
-        const bool in = live && n < N;
-        A2[i] = in ? a.A[(int64_t)c * N + n] * 1.4426950408889634f : 0.f;
+        A2[i] *= kScLog2e;
         S[i] = 0.f;
     }
     if constexpr (MODE == kScSummary) {
         if (last_seg == 0) return;                               // nobody folds
         if (seg == last_seg) {                                   // the start state is handed on from here: the second launch
-            float* dst = a.seg_state + (((int64_t)b * a.nseg + seg) * C + c) * N;      // overwrites the slot
-#pragma unroll
-            for (int i = 0; i < SPL; ++i) {
-                const int n = sub * SPL + i;
-                if (live && n < N) dst[n] = start > 0 ? slot_state[n] : 0.f;
-            }
+            if (!live) return;                                   // overwrites the slot
+            sc_load_states<SPL>(slot_state, n0, N, start > 0, S);
+            sc_store_states<SPL>(a.seg_state + (((int64_t)b * a.nseg + seg) * C + c) * N, n0, N, S);
             return;
         }
     } else {
-        const float* src = slot_state;
-        bool have = start > 0;
-        if constexpr (MODE == kScFinal) {
-            if (last_seg > 0) {
-                src = a.seg_state + (((int64_t)b * a.nseg + last_seg) * C + c) * N;
-                have = true;
-            }
-        }
-#pragma unroll
-        for (int i = 0; i < SPL; ++i) {
-            const int n = sub * SPL + i;
-            if (have && live && n < N) S[i] = src[n];
-        }
-        if constexpr (MODE == kScFinal) {
+        if (MODE == kScFinal && last_seg > 0) {
+            sc_load_states<SPL>(a.seg_state + (((int64_t)b * a.nseg + last_seg) * C + c) * N, n0, N, live, S);
             for (int s = 0; s < seg; ++s) {
                 const int64_t at = ((int64_t)b * a.nseg + s) * C + c;
                 const float dsum = live ? a.seg_dt[at] : 0.f;
+                float loc[SPL];
+                sc_load_states<SPL>(a.seg_state + at * N, n0, N, live, loc);
 #pragma unroll
-                for (int i = 0; i < SPL; ++i) {
-                    const int n = sub * SPL + i;
-                    if (live && n < N) S[i] = __builtin_amdgcn_exp2f(dsum * A2[i]) * S[i] + a.seg_state[at * N + n];
-                }
+                for (int i = 0; i < SPL; ++i) S[i] = __builtin_amdgcn_exp2f(dsum * A2[i]) * S[i] + loc[i];
             }
+        } else {
+            sc_load_states<SPL>(slot_state, n0, N, live && start > 0, S);
         }
     }
     float dt_sum = 0.f;
@@ -241,18 +268,42 @@ __global__ __launch_bounds__(kScThreads) void selective_scan_kernel(const ScArgs
     if constexpr (MODE == kScSummary) {
         const int64_t at = ((int64_t)b * a.nseg + seg) * C + c;
         if (sub == 0) a.seg_dt[at] = dt_sum;
-#pragma unroll
-        for (int i = 0; i < SPL; ++i) {
-            const int n = sub * SPL + i;
-            if (n < N) a.seg_state[at * N + n] = S[i];
-        }
+        sc_store_states<SPL>(a.seg_state + at * N, n0, N, S);
     } else if (seg == last_seg) {
-#pragma unroll
-        for (int i = 0; i < SPL; ++i) {
-            const int n = sub * SPL + i;
-            if (n < N) slot_state[n] = S[i];
-        }
+        sc_store_states<SPL>(slot_state, n0, N, S);
     }
+}
+
+// One token per sequence: nothing is worth preparing, every lane reads what it needs.
+template <typename T, int L, int SPL>
+__global__ __launch_bounds__(kScThreads) void selective_scan_single_kernel(const ScArgs<T> a) {
+    constexpr int CPB = kScThreads / L;
+    const int b = blockIdx.x, t = a.cu_q[b];
+    if (a.cu_q[b + 1] - t != 1) return;
+    const bool fresh = a.cu_k[b + 1] - a.cu_k[b] == 1;
+    const int ch = threadIdx.x / L, sub = threadIdx.x % L, c = blockIdx.y * CPB + ch, C = a.C, N = a.N, n0 = sub * SPL;
+    const bool live = c < C;
+    const int cc = live ? c : C - 1;
+    float* slot_state = a.state + ((int64_t)a.slots[b] * C + cc) * N;
+    float A[SPL], S[SPL];
+    sc_load_states<SPL>(slot_state, n0, N, live && !fresh, S);
+    sc_load_states<SPL>(a.A + (int64_t)cc * N, n0, N, live, A);
+    const float x = (float)a.x[(int64_t)t * a.x_stride + cc], z = (float)a.z[(int64_t)t * a.z_stride + cc];
+    const float dt = sc_softplus((float)a.dt_raw[(int64_t)t * a.dt_stride + cc] + a.dt_bias[cc]);
+    const T *bp = a.Bm + (int64_t)t * a.b_stride, *cp = a.Cm + (int64_t)t * a.c_stride;
+    const float dx = dt * x, dt2 = dt * kScLog2e;
+    float y = 0.f;
+#pragma unroll
+    for (int i = 0; i < SPL; ++i) {
+        const int n = n0 + i;
+        const float bn = n < N ? (float)bp[n] : 0.f, cn = n < N ? (float)cp[n] : 0.f;
+        S[i] = __builtin_amdgcn_exp2f(dt2 * A[i]) * S[i] + dx * bn;
+        y += S[i] * cn;
+    }
+    y = sc_group_sum<L>(y);
+    if (!live) return;
+    sc_store_states<SPL>(slot_state, n0, N, S);
+    if (sub == 0) a.out[(int64_t)t * a.out_stride + c] = (T)((y + a.D[c] * x) * sc_silu(z));
 }
 
 struct ScPlan {
@@ -264,6 +315,10 @@ struct ScPlan {
 static ScPlan sc_plan(int B, int C, int N, int max_seqlen_q) {
     ScPlan p{1, 4, 1, 0, 0};
     while (p.L * 4 < N) p.L *= 2;
+    if (max_seqlen_q == 1) {
+        p.seg_len = 1;
+        return p;
+    }
     // eight states per lane (half the lanes, less work per token beside the states) when there are plenty of waves
     if (p.L >= 4 && (int64_t)B * C * p.L / 64 >= 8192) {
         p.SPL = 8;
@@ -288,6 +343,10 @@ template <typename T, int L, int SPL>
 static void launch_scan(const ScArgs<T>& a, int B, hipStream_t s) {
     constexpr int CPB = kScThreads / L;
     const dim3 grid((unsigned)B, (unsigned)((a.C + CPB - 1) / CPB), (unsigned)a.nseg), block(kScThreads);
+    if (a.seg_len == 1) {                                        // (max_seqlen_q == 1)
+        hipLaunchKernelGGL((selective_scan_single_kernel<T, L, SPL>), grid, block, 0, s, a);
+        return;
+    }
     if (a.nseg == 1) {
         hipLaunchKernelGGL((selective_scan_kernel<T, L, SPL, kScWhole>), grid, block, 0, s, a);
         return;

@@ -79,4 +79,4 @@ class FixedDecayMemory(nn.Module):
         """q, k: [T, H, Dk]; v: [T, H, Dv] as projected; returns [T, H * Dv] float32."""
         ctx = get_context()
         return ops.fixed_decay_memory(q, k, v, self.decay, cache["state"], ctx.cu_seqlens_q, ctx.cu_seqlens_k, ctx.state_slots,
-                                      ctx.max_seqlen_q, ctx.min_seqlen_q)
+                                      ctx.max_seqlen_q, ctx.portion_kinds)

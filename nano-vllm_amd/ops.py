@@ -1582,11 +1582,23 @@ def selective_scan(x: torch.Tensor, dt_raw: torch.Tensor, z: torch.Tensor, Bm: t
     return out
 
 
+FEW_ROWS = 16                      # NV_FEW_ROWS
+
+
+def portion_kinds(rows) -> int:
+    """NV_PORTION_* of a step from its sequences' row counts (host numbers): 1 single tokens, 2 up to FEW_ROWS, 4 more."""
+    kinds = 0
+    for n in rows:
+        kinds |= 0 if n <= 0 else 1 if n == 1 else 2 if n <= FEW_ROWS else 4
+    return kinds
+
+
 def fixed_decay_memory(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor, state: torch.Tensor,
                        cu_seqlens_q: torch.Tensor, cu_seqlens_k: torch.Tensor, state_slots: torch.Tensor, max_seqlen_q: int,
-                       min_seqlen_q: int = 0) -> torch.Tensor:
+                       portions: int = 7) -> torch.Tensor:
     """S <- decay_h S + silu(k) silu(v)^T, o = S^T silu(q) over a step's rows; q, k: [T, H, Dk]; v: [T, H, Dv] as projected;
-    decay [H] float32; state [slots, H, Dk, Dv] float32 updated in place; returns o as float32 [T, H * Dv]."""
+    decay [H] float32; state [slots, H, Dk, Dv] float32 updated in place; returns o as float32 [T, H * Dv].  portions: the kinds
+    of portions in the step (`portion_kinds`; 7: not known)."""
     dt = _dt(q, "q")
     T, H, Dk = q.shape
     Dv = v.shape[2]
@@ -1607,7 +1619,7 @@ def fixed_decay_memory(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay:
     rc = dll.nv_fixed_decay_memory(q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0), k.stride(0), v.stride(0),
                                    _f32c(decay, "decay"), state.data_ptr(), out.data_ptr(), out.stride(0),
                                    cu_seqlens_q.data_ptr(), cu_seqlens_k.data_ptr(), state_slots.data_ptr(), B, H, Dk, Dv, mq,
-                                   int(min_seqlen_q), dt, _ptr(ws), ws.numel() if ws is not None else 0, _stream(q))
+                                   int(portions), dt, _ptr(ws), ws.numel() if ws is not None else 0, _stream(q))
     _lib.check(rc, "nv_fixed_decay_memory", dll)
     return out
 

@@ -56,9 +56,9 @@ class CacheContext:
     # Extension (optional): host copy (numpy int32 [B+1]) of cu_seqlens_q, for layers that lay out their launch per
     # sequence on the host (layers/chunk_attention.py cuts prompt portions into row tiles).
     cu_seqlens_q_host: Optional[object] = None
-    # Extension (optional): the fewest query tokens a sequence of the step has (0 = unknown), for layers with one launch for
-    # short and one for long portions (layers/gated_memory.py).
-    min_seqlen_q: int = 0
+    # Extension (optional): which kinds of portions the step holds (`ops.portion_kinds`), for layers with a launch for each
+    # (layers/gated_memory.py).
+    portion_kinds: int = 7
 
 
 _cache_context: ContextVar[Optional[CacheContext]] = ContextVar("CacheContext", default=None)

@@ -38,7 +38,7 @@ N_Q, N_K, SLOTS = [5, 1, 17, 2, 64, 131, 1], [5, 40, 30, 2, 64, 140, 9], [2, 0, 
 
 def set_step(n_q, n_k, slots):
     ctx, pos = paged_context(n_q, n_k, 8, sum(-(-n // 8) for n in n_k) + 4, 1, DEV, slots=slots)
-    ctx.max_seqlen_q, ctx.min_seqlen_q = max(n_q), min(n_q)
+    ctx.portion_kinds = nv.ops.portion_kinds(n_q)
     nv.set_context(ctx)
     return sum(n_q), pos
 

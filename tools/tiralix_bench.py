@@ -71,7 +71,7 @@ def kernel_records(dev):
     for name, n_qs in cases.items():
         note("recurrent kernels, " + name)
         ctx, pos, _ = paged(n_qs, [n + 100 for n in n_qs], bs, dev)
-        ctx.min_seqlen_q = min(n_qs)
+        ctx.portion_kinds = ops.portion_kinds(n_qs)
         T, B = sum(n_qs), len(n_qs)
         nv.set_context(ctx)
         rec = {}
