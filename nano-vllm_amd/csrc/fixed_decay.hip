@@ -41,7 +41,6 @@ struct FdParams {
     FixedDecayArgs f;
     int seg_len, nseg;                         // tokens per segment (a multiple of kFdChunk)
     float* seg_state;                          // [B, nseg, H, Dk, Dv]
-    int vec_qk, vec_v, vec_o;
 };
 
 __device__ __forceinline__ float fd_silu(float x) {
@@ -50,6 +49,18 @@ __device__ __forceinline__ float fd_silu(float x) {
 __device__ __forceinline__ uint4 fd_silu8(uint4 u) {
     return make_uint4(pack_bf16(fd_silu(bf16_lo(u.x)), fd_silu(bf16_hi(u.x))), pack_bf16(fd_silu(bf16_lo(u.y)), fd_silu(bf16_hi(u.y))),
                       pack_bf16(fd_silu(bf16_lo(u.z)), fd_silu(bf16_hi(u.z))), pack_bf16(fd_silu(bf16_lo(u.w)), fd_silu(bf16_hi(u.w))));
+}
+// 8 columns of a row from c0 on, zeros past `cols` or for a missing row.  One guarded load and nothing else in the whole-piece
+// form: a choice between two forms at run time would make every load wait for the one before.
+template <bool VEC>
+__device__ __forceinline__ uint4 fd_fetch(const __bf16* row, int c0, int cols) {
+    if constexpr (VEC) {
+        uint4 r = make_uint4(0, 0, 0, 0);
+        if (row != nullptr && c0 < cols) r = *(const uint4*)(row + c0);
+        return r;
+    } else {
+        return tile_fetch<__bf16>(row, c0, cols, false);
+    }
 }
 // x = hi + lo, each bf16
 __device__ __forceinline__ void fd_split(const float* x, bf16x8& hi, bf16x8& lo) {
@@ -79,7 +90,8 @@ __device__ __forceinline__ f32x4 fd_mma(bf16x8 a, bf16x8 b, f32x4 c) {
 
 enum { kFdWhole = 0, kFdSummary = 1, kFdFinal = 2 };
 
-template <int DKT, int MODE>
+// VEC: rows of q, k, v may be read and rows of out written in 16-byte pieces.
+template <int DKT, int MODE, bool VEC>
 __global__ __launch_bounds__(256) void fixed_decay_chunk_kernel(const FdParams p) {
     constexpr int DK = 32 * DKT, QS = DK + 8;
     extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
@@ -108,37 +120,46 @@ __global__ __launch_bounds__(256) void fixed_decay_chunk_kernel(const FdParams p
     for (int t = 0; t < 2 * DKT; ++t)
 #pragma unroll
         for (int r = 0; r < 4; ++r) S[t][r] = 0.f;
-    auto each_state = [&](auto&& fn) {
+    // Entries outside the state are read from its edge and not written: all loads of a state are in flight together.
+    auto load_state = [&](const float* m, f32x4* to) {
+#pragma unroll
+        for (int t = 0; t < 2 * DKT; ++t)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) to[t][r] = m[(int64_t)min(16 * t + 4 * g + r, Dk - 1) * Dv + min(col, Dv - 1)];
+    };
+    auto store_state = [&](float* m) {
 #pragma unroll
         for (int t = 0; t < 2 * DKT; ++t)
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const int d = 16 * t + 4 * g + r;
-                if (d < Dk && col < Dv) fn(t, r, (int64_t)d * Dv + col);
+                if (d < Dk && col < Dv) m[(int64_t)d * Dv + col] = S[t][r];
             }
     };
     if constexpr (MODE == kFdSummary) {
         if (last_seg == 0) return;                               // nobody folds
         if (seg == last_seg) {                                   // the start state is handed on from here: the second launch
-            float* dst = seg_at(seg);                            // overwrites the slot
-            each_state([&](int, int, int64_t at) { dst[at] = start > 0 ? slot_state[at] : 0.f; });
+            if (start > 0) load_state(slot_state, S);            // overwrites the slot
+            store_state(seg_at(seg));
             return;
         }
     } else {
-        const float* src = slot_state;
-        bool have = start > 0;
         if (MODE == kFdFinal && last_seg > 0) {
-            src = seg_at(last_seg);
-            have = true;
-        }
-        if (have) each_state([&](int t, int r, int64_t at) { S[t][r] = src[at]; });
-        if constexpr (MODE == kFdFinal) {
+            load_state(seg_at(last_seg), S);
             const float over = powf(decay, (float)p.seg_len);
+            f32x4 loc[2 * DKT];
             for (int s = 0; s < seg; ++s) {
-                const float* loc = seg_at(s);
-                each_state([&](int t, int r, int64_t at) { S[t][r] = over * S[t][r] + loc[at]; });
+                load_state(seg_at(s), loc);
+#pragma unroll
+                for (int t = 0; t < 2 * DKT; ++t)
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) S[t][r] = over * S[t][r] + loc[t][r];
             }
+        } else if (start > 0) {
+            load_state(slot_state, S);
         }
+        // (what stands for entries outside the state meets zeros in k and is never read out: q is zero there, and so is the
+        // value column's output not written)
     }
     if (tid <= kFdChunk) pw[tid] = powf(decay, (float)tid);
     const int stop = seg == last_seg ? len_q : first + p.seg_len;
@@ -151,15 +172,15 @@ __global__ __launch_bounds__(256) void fixed_decay_chunk_kernel(const FdParams p
             const int64_t t = q0 + t0 + row;
             const bool in = t0 + row < stop;
             if constexpr (MODE != kFdSummary)
-                rq[i] = tile_fetch<__bf16>(in ? (const __bf16*)f.q + t * f.q_stride + (int64_t)h * Dk : nullptr, d0, Dk, p.vec_qk);
-            rk[i] = tile_fetch<__bf16>(in ? (const __bf16*)f.k + t * f.k_stride + (int64_t)h * Dk : nullptr, d0, Dk, p.vec_qk);
+                rq[i] = fd_fetch<VEC>(in ? (const __bf16*)f.q + t * f.q_stride + (int64_t)h * Dk : nullptr, d0, Dk);
+            rk[i] = fd_fetch<VEC>(in ? (const __bf16*)f.k + t * f.k_stride + (int64_t)h * Dk : nullptr, d0, Dk);
         }
 #pragma unroll
         for (int i = 0; i < 2; ++i) {
             const int pc = tid + 256 * i, row = pc >> 3, c0 = cg * 64 + (pc & 7) * 8;
             const bool in = t0 + row < stop;
-            rv[i] = tile_fetch<__bf16>(in ? (const __bf16*)f.v + (int64_t)(q0 + t0 + row) * f.v_stride + (int64_t)h * Dv : nullptr,
-                                       c0, Dv, p.vec_v);
+            rv[i] = fd_fetch<VEC>(in ? (const __bf16*)f.v + (int64_t)(q0 + t0 + row) * f.v_stride + (int64_t)h * Dv : nullptr,
+                                       c0, Dv);
         }
     };
     fetch(first);
@@ -251,7 +272,7 @@ __global__ __launch_bounds__(256) void fixed_decay_chunk_kernel(const FdParams p
                 const int i = 16 * it + l15, c = cg * 64 + 16 * wave + 4 * g;
                 if (i < nt && c < Dv) {
                     float* dst = f.out + (int64_t)(q0 + t0 + i) * f.out_stride + (int64_t)h * Dv + c;
-                    if (p.vec_o) {
+                    if constexpr (VEC) {
                         *(float4*)dst = make_float4(o[it][0], o[it][1], o[it][2], o[it][3]);
                     } else {
 #pragma unroll
@@ -285,10 +306,8 @@ __global__ __launch_bounds__(256) void fixed_decay_chunk_kernel(const FdParams p
             }
         }
     }
-    if (MODE == kFdSummary || seg == last_seg) {
-        float* dst = MODE == kFdSummary ? seg_at(seg) : slot_state;
-        each_state([&](int t, int r, int64_t at) { dst[at] = S[t][r]; });
-    }
+    if (MODE == kFdSummary) store_state(seg_at(seg));
+    else if (seg == last_seg) store_state(slot_state);
 }
 
 // ------------------------------------------------------------------------------------------------ one token
@@ -392,16 +411,18 @@ static FdPlan fd_plan(int B, int H, int Dk, int Dv, int max_seqlen_q) {
 }
 
 template <int DKT>
-static void launch_chunks(const FdParams& p, hipStream_t s) {
+static void launch_chunks(const FdParams& p, bool vec, hipStream_t s) {
     const size_t lds = sizeof(__bf16) * (2 * kFdChunk * (32 * DKT + 8) + kFdChunk * kFdVs) + sizeof(bf16x8) * 4 * 2 * 2 * 64 +
                        sizeof(float) * (kFdChunk + 1);
     const dim3 grid((unsigned)p.f.num_seqs, (unsigned)(p.f.H * ((p.f.Dv + 63) / 64)), (unsigned)p.nseg), block(256);
-    if (p.nseg == 1) {
-        hipLaunchKernelGGL((fixed_decay_chunk_kernel<DKT, kFdWhole>), grid, block, lds, s, p);
-        return;
+    if (!vec) {                                                  // rows of odd sizes: one plain form (the plan has one segment)
+        hipLaunchKernelGGL((fixed_decay_chunk_kernel<DKT, kFdWhole, false>), grid, block, lds, s, p);
+    } else if (p.nseg == 1) {
+        hipLaunchKernelGGL((fixed_decay_chunk_kernel<DKT, kFdWhole, true>), grid, block, lds, s, p);
+    } else {
+        hipLaunchKernelGGL((fixed_decay_chunk_kernel<DKT, kFdSummary, true>), grid, block, lds, s, p);
+        hipLaunchKernelGGL((fixed_decay_chunk_kernel<DKT, kFdFinal, true>), grid, block, lds, s, p);
     }
-    hipLaunchKernelGGL((fixed_decay_chunk_kernel<DKT, kFdSummary>), grid, block, lds, s, p);
-    hipLaunchKernelGGL((fixed_decay_chunk_kernel<DKT, kFdFinal>), grid, block, lds, s, p);
 }
 
 }  // namespace nv
@@ -447,15 +468,14 @@ extern "C" int nv_fixed_decay_memory(const void* q, const void* k, const void* v
     NV_REQUIRE(plan.ws_floats == 0 || (workspace && workspace_bytes >= plan.ws_floats * (int64_t)sizeof(float)), NV_ERR_WORKSPACE,
                "nv_fixed_decay_memory: workspace of %lld bytes, need %lld", (long long)workspace_bytes,
                (long long)(plan.ws_floats * (int64_t)sizeof(float)));
-    p.nseg = plan.nseg;
+    const bool vec = Dk % 8 == 0 && Dv % 8 == 0 && q_stride % 8 == 0 && k_stride % 8 == 0 && v_stride % 8 == 0 && out_stride % 4 == 0 &&
+                     ((uintptr_t)q | (uintptr_t)k | (uintptr_t)v | (uintptr_t)out) % 16 == 0;
+    p.nseg = vec ? plan.nseg : 1;
     p.seg_len = plan.seg_len;
     p.seg_state = (float*)workspace;
-    p.vec_qk = Dk % 8 == 0 && q_stride % 8 == 0 && k_stride % 8 == 0 && ((uintptr_t)q | (uintptr_t)k) % 16 == 0;
-    p.vec_v = Dv % 8 == 0 && v_stride % 8 == 0 && (uintptr_t)v % 16 == 0;
-    p.vec_o = Dv % 4 == 0 && out_stride % 4 == 0 && (uintptr_t)out % 16 == 0;
-    if (Dk <= 32) launch_chunks<1>(p, s);
-    else if (Dk <= 64) launch_chunks<2>(p, s);
-    else if (Dk <= 96) launch_chunks<3>(p, s);
-    else launch_chunks<4>(p, s);
+    if (Dk <= 32) launch_chunks<1>(p, vec, s);
+    else if (Dk <= 64) launch_chunks<2>(p, vec, s);
+    else if (Dk <= 96) launch_chunks<3>(p, vec, s);
+    else launch_chunks<4>(p, vec, s);
     return check_launch("nv_fixed_decay_memory");
 }

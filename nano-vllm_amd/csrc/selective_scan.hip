@@ -95,31 +95,47 @@ struct ScArgs {
     int C, N;
     int seg_len, nseg;                         // tokens per segment (a multiple of kScTile), segments of the longest sequence
     float *seg_state, *seg_dt;                 // [B, nseg, C, N], [B, nseg, C]
-    int vec;                                   // rows of x, dt_raw, z, out may be walked in pieces of four columns
 };
 
-// Four neighbouring columns of a row, zeros from `cols` on.
-template <typename T>
-__device__ __forceinline__ Cols<4> sc_load4(const T* row, int c, int cols, bool vec) {
-    if (vec) return row_load<4>(row + c);
-    Cols<4> o;
+// Four neighbouring columns of a row as they lie in memory (zeros from `cols` on): what is on its way must not be touched.
+template <typename T> struct ScRaw;
+template <> struct ScRaw<__bf16> { typedef uint2 type; };
+template <> struct ScRaw<float> { typedef float4 type; };
+template <bool VEC, typename T>
+__device__ __forceinline__ typename ScRaw<T>::type sc_fetch4(const T* row, int c, int cols, bool in) {
+    typedef typename ScRaw<T>::type R;
+    R r = {};
+    if (in) {
+        if constexpr (VEC) {
+            r = *(const R*)(row + c);
+        } else {
+            T* e = (T*)&r;
 #pragma unroll
-    for (int e = 0; e < 4; ++e) o.v[e] = c + e < cols ? (float)row[c + e] : 0.f;
-    return o;
+            for (int i = 0; i < 4; ++i)
+                if (c + i < cols) e[i] = row[c + i];
+        }
+    }
+    return r;
 }
+__device__ __forceinline__ Cols<4> sc_widen(uint2 r) {
+    return Cols<4>{{bf16_lo(r.x), bf16_hi(r.x), bf16_lo(r.y), bf16_hi(r.y)}};
+}
+__device__ __forceinline__ Cols<4> sc_widen(float4 r) { return Cols<4>{{r.x, r.y, r.z, r.w}}; }
 
 enum { kScWhole = 0, kScSummary = 1, kScFinal = 2 };
 
-template <typename T, int L, int SPL, int MODE>
+// VEC: rows of x, dt_raw, z, out, B and C may be walked in pieces of four columns.
+template <typename T, int L, int SPL, int MODE, bool VEC>
 __global__ __launch_bounds__(kScThreads) void selective_scan_kernel(const ScArgs<T> a) {
     constexpr int CPB = kScThreads / L;                          // channels of the workgroup
     constexpr int NP = L * SPL;                                  // states, padded
     constexpr int PIECES = kScTile * CPB / 4;                    // four-channel pieces of a tile
     constexpr int IT = (PIECES + kScThreads - 1) / kScThreads;
-    constexpr int IB = (kScTile * NP + kScThreads - 1) / kScThreads;
+    constexpr int BPIECES = kScTile * NP / 4;                    // four-state pieces of B and of C
+    constexpr int IB = (BPIECES + kScThreads - 1) / kScThreads;
     __shared__ float2 dts[kScTile][CPB];                         // (dt, dt x)
-    __shared__ float bs[kScTile][NP], cs[kScTile][NP];
-    __shared__ float ys[kScTile][CPB];
+    __shared__ __attribute__((aligned(16))) float bs[kScTile][NP], cs[kScTile][NP];
+    __shared__ __attribute__((aligned(16))) float ys[kScTile][CPB];
     const int b = blockIdx.x, c0 = blockIdx.y * CPB, seg = blockIdx.z;
     const int q0 = a.cu_q[b], len_q = a.cu_q[b + 1] - q0;
     if (len_q <= 0) return;
@@ -162,30 +178,34 @@ __global__ __launch_bounds__(kScThreads) void selective_scan_kernel(const ScArgs
         }
     }
     float dt_sum = 0.f;
+    // the thread's four channels wherever it prepares or writes tokens (the threads are whole rows of pieces)
+    const int cl = (tid % (CPB / 4)) * 4, cc = c0 + cl;
+    float bias[4], skip[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+        bias[e] = cc + e < C ? a.dt_bias[cc + e] : 0.f;
+        skip[e] = cc + e < C ? a.D[cc + e] : 0.f;
+    }
     const int stop = seg == last_seg ? len_q : first + a.seg_len;
-    // registers of the tile that comes next, and (x, z) of the one that is being scanned
-    Cols<4> ndt[IT], nx[IT], nz[IT], x_cur[IT], z_cur[IT];
-    float nb[IB], nc[IB];
+    // the tile that comes next, as it arrives, and (x, z) of the one that is being scanned
+    typename ScRaw<T>::type ndt[IT], nx[IT], nz[IT], x_cur[IT], z_cur[IT], nb[IB], nc[IB];
     auto fetch = [&](int t0) {
 #pragma unroll
         for (int k = 0; k < IT; ++k) {
-            const int p = tid + k * kScThreads, tt = p / (CPB / 4), cc = c0 + (p % (CPB / 4)) * 4;
-            if (p < PIECES && t0 + tt < stop && cc < C) {
-                const int64_t t = q0 + t0 + tt;
-                ndt[k] = sc_load4(a.dt_raw + t * a.dt_stride, cc, C, a.vec);
-                nx[k] = sc_load4(a.x + t * a.x_stride, cc, C, a.vec);
-                if constexpr (MODE != kScSummary) nz[k] = sc_load4(a.z + t * a.z_stride, cc, C, a.vec);
-            } else {
-#pragma unroll
-                for (int e = 0; e < 4; ++e) ndt[k].v[e] = nx[k].v[e] = nz[k].v[e] = 0.f;
-            }
+            const int p = tid + k * kScThreads, tt = p / (CPB / 4);
+            const bool in = p < PIECES && t0 + tt < stop && cc < C;
+            const int64_t t = q0 + t0 + tt;
+            ndt[k] = sc_fetch4<VEC>(a.dt_raw + t * a.dt_stride, cc, C, in);
+            nx[k] = sc_fetch4<VEC>(a.x + t * a.x_stride, cc, C, in);
+            if constexpr (MODE != kScSummary) nz[k] = sc_fetch4<VEC>(a.z + t * a.z_stride, cc, C, in);
         }
 #pragma unroll
         for (int k = 0; k < IB; ++k) {
-            const int p = tid + k * kScThreads, tt = p / NP, n = p % NP;
-            const bool in = tt < kScTile && t0 + tt < stop && n < N;
-            nb[k] = in ? (float)a.Bm[(int64_t)(q0 + t0 + tt) * a.b_stride + n] : 0.f;
-            if constexpr (MODE != kScSummary) nc[k] = in ? (float)a.Cm[(int64_t)(q0 + t0 + tt) * a.c_stride + n] : 0.f;
+            const int p = tid + k * kScThreads, tt = p / (NP / 4), n = (p % (NP / 4)) * 4;
+            const bool in = p < BPIECES && t0 + tt < stop && n < N;
+            const int64_t t = q0 + t0 + tt;
+            nb[k] = sc_fetch4<VEC>(a.Bm + t * a.b_stride, n, N, in);
+            if constexpr (MODE != kScSummary) nc[k] = sc_fetch4<VEC>(a.Cm + t * a.c_stride, n, N, in);
         }
     };
     fetch(first);
@@ -194,24 +214,25 @@ __global__ __launch_bounds__(kScThreads) void selective_scan_kernel(const ScArgs
         __syncthreads();                                         // the previous tile has been scanned and written
 #pragma unroll
         for (int k = 0; k < IT; ++k) {
-            const int p = tid + k * kScThreads, tt = p / (CPB / 4), cl = (p % (CPB / 4)) * 4;
+            const int p = tid + k * kScThreads, tt = p / (CPB / 4);
             x_cur[k] = nx[k];
-            z_cur[k] = nz[k];
+            if constexpr (MODE != kScSummary) z_cur[k] = nz[k];
             if (p < PIECES) {
+                const Cols<4> dr = sc_widen(ndt[k]), xr = sc_widen(nx[k]);
 #pragma unroll
                 for (int e = 0; e < 4; ++e) {
                     // (dt = 0 behind the portion's end: those steps leave the state as it is)
-                    const float dt = tt < nt && c0 + cl + e < C ? sc_softplus(ndt[k].v[e] + a.dt_bias[c0 + cl + e]) : 0.f;
-                    dts[tt][cl + e] = make_float2(dt, dt * nx[k].v[e]);
+                    const float dt = tt < nt ? sc_softplus(dr.v[e] + bias[e]) : 0.f;
+                    dts[tt][cl + e] = make_float2(dt, dt * xr.v[e]);
                 }
             }
         }
 #pragma unroll
         for (int k = 0; k < IB; ++k) {
-            const int p = tid + k * kScThreads, tt = p / NP, n = p % NP;
-            if (tt < kScTile) {
-                bs[tt][n] = nb[k];
-                if constexpr (MODE != kScSummary) cs[tt][n] = nc[k];
+            const int p = tid + k * kScThreads, tt = p / (NP / 4), n = (p % (NP / 4)) * 4;
+            if (p < BPIECES) {
+                row_store<4>(&bs[tt][n], sc_widen(nb[k]));
+                if constexpr (MODE != kScSummary) row_store<4>(&cs[tt][n], sc_widen(nc[k]));
             }
         }
         __syncthreads();
@@ -245,16 +266,14 @@ __global__ __launch_bounds__(kScThreads) void selective_scan_kernel(const ScArgs
             __syncthreads();
 #pragma unroll
             for (int k = 0; k < IT; ++k) {
-                const int p = tid + k * kScThreads, tt = p / (CPB / 4), cl = (p % (CPB / 4)) * 4, cc = c0 + cl;
+                const int p = tid + k * kScThreads, tt = p / (CPB / 4);
                 if (p >= PIECES || tt >= nt || cc >= C) continue;
+                const Cols<4> xr = sc_widen(x_cur[k]), zr = sc_widen(z_cur[k]);
                 Cols<4> o;
 #pragma unroll
-                for (int e = 0; e < 4; ++e) {
-                    const float skip = cc + e < C ? a.D[cc + e] : 0.f;
-                    o.v[e] = (ys[tt][cl + e] + skip * x_cur[k].v[e]) * sc_silu(z_cur[k].v[e]);
-                }
+                for (int e = 0; e < 4; ++e) o.v[e] = (ys[tt][cl + e] + skip[e] * xr.v[e]) * sc_silu(zr.v[e]);
                 T* dst = a.out + (int64_t)(q0 + t0 + tt) * a.out_stride + cc;
-                if (a.vec) {
+                if constexpr (VEC) {
                     row_store<4>(dst, o);
                 } else {
 #pragma unroll
@@ -324,12 +343,11 @@ static ScPlan sc_plan(int B, int C, int N, int max_seqlen_q) {
         p.SPL = 8;
         p.L /= 2;
     }
-    const int cpb = kScThreads / p.L;
-    const int64_t waves = (int64_t)B * ((C + cpb - 1) / cpb) * (kScThreads / 64);
+    const int64_t waves = (int64_t)B * C * p.L / 64;
     const int mq = std::max(1, max_seqlen_q);
     p.seg_len = (mq + kScTile - 1) / kScTile * kScTile;
-    if (waves < 1024 && mq >= 256) {
-        const int want = (int)std::min<int64_t>((2048 + waves - 1) / waves, 16);
+    if (waves < 2048 && mq >= 256) {
+        const int want = (int)std::min<int64_t>((4096 + waves - 1) / waves, 16);
         const int most = mq / 128;
         p.nseg = std::max(1, std::min(want, most));
         p.seg_len = ((mq + p.nseg - 1) / p.nseg + kScTile - 1) / kScTile * kScTile;
@@ -343,26 +361,50 @@ template <typename T, int L, int SPL>
 static void launch_scan(const ScArgs<T>& a, int B, hipStream_t s) {
     constexpr int CPB = kScThreads / L;
     const dim3 grid((unsigned)B, (unsigned)((a.C + CPB - 1) / CPB), (unsigned)a.nseg), block(kScThreads);
-    if (a.seg_len == 1) {                                        // (max_seqlen_q == 1)
-        hipLaunchKernelGGL((selective_scan_single_kernel<T, L, SPL>), grid, block, 0, s, a);
-        return;
-    }
     if (a.nseg == 1) {
-        hipLaunchKernelGGL((selective_scan_kernel<T, L, SPL, kScWhole>), grid, block, 0, s, a);
+        hipLaunchKernelGGL((selective_scan_kernel<T, L, SPL, kScWhole, true>), grid, block, 0, s, a);
         return;
     }
-    hipLaunchKernelGGL((selective_scan_kernel<T, L, SPL, kScSummary>), grid, block, 0, s, a);
-    hipLaunchKernelGGL((selective_scan_kernel<T, L, SPL, kScFinal>), grid, block, 0, s, a);
+    hipLaunchKernelGGL((selective_scan_kernel<T, L, SPL, kScSummary, true>), grid, block, 0, s, a);
+    hipLaunchKernelGGL((selective_scan_kernel<T, L, SPL, kScFinal, true>), grid, block, 0, s, a);
 }
 
 template <typename T>
-static int run_scan(const ScArgs<T>& a, const ScPlan& p, int B, hipStream_t s) {
-#define NV_SC(LL, SS) \
-    if (p.L == LL && p.SPL == SS) { launch_scan<T, LL, SS>(a, B, s); return check_launch("nv_selective_scan"); }
+static int run_scan(ScArgs<T> a, const ScPlan& p, bool vec, int B, hipStream_t s) {
+    int L = p.L, SPL = p.SPL;
+    const bool single = a.seg_len == 1;                          // (max_seqlen_q == 1)
+    if (!single && !vec) {                                       // rows of odd sizes: one plain form
+        L = L * SPL / 4;
+        SPL = 4;
+        a.nseg = 1;
+    }
+#define NV_SC_SINGLE(LL)                                                                                                       \
+    if (single && L == LL) {                                                                                                    \
+        constexpr int CPS = kScThreads / LL;                                                                              \
+        hipLaunchKernelGGL((selective_scan_single_kernel<T, LL, 4>), dim3((unsigned)B, (unsigned)((a.C + CPS - 1) / CPS)),       \
+                           dim3(kScThreads), 0, s, a);                                                                    \
+        return check_launch("nv_selective_scan");                                                                               \
+    }
+#define NV_SC(LL, SS)                                                                                                          \
+    if (!single && vec && L == LL && SPL == SS) {                                                                               \
+        launch_scan<T, LL, SS>(a, B, s);                                                                                        \
+        return check_launch("nv_selective_scan");                                                                               \
+    }
+#define NV_SC_PLAIN(LL)                                                                                                        \
+    if (!single && !vec && L == LL) {                                                                                           \
+        constexpr int CPB = kScThreads / LL;                                                                                \
+        hipLaunchKernelGGL((selective_scan_kernel<T, LL, 4, kScWhole, false>), dim3((unsigned)B, (unsigned)((a.C + CPB - 1) / CPB)), \
+                           dim3(kScThreads), 0, s, a);                                                                      \
+        return check_launch("nv_selective_scan");                                                                               \
+    }
+    NV_SC_SINGLE(1) NV_SC_SINGLE(2) NV_SC_SINGLE(4) NV_SC_SINGLE(8) NV_SC_SINGLE(16) NV_SC_SINGLE(32) NV_SC_SINGLE(64)
     NV_SC(1, 4) NV_SC(2, 4) NV_SC(4, 4) NV_SC(8, 4) NV_SC(16, 4) NV_SC(32, 4) NV_SC(64, 4)
     NV_SC(2, 8) NV_SC(4, 8) NV_SC(8, 8) NV_SC(16, 8) NV_SC(32, 8)
+    NV_SC_PLAIN(1) NV_SC_PLAIN(2) NV_SC_PLAIN(4) NV_SC_PLAIN(8) NV_SC_PLAIN(16) NV_SC_PLAIN(32) NV_SC_PLAIN(64)
+#undef NV_SC_SINGLE
 #undef NV_SC
-    set_error("nv_selective_scan: no kernel for %d lanes x %d states", p.L, p.SPL);
+#undef NV_SC_PLAIN
+    set_error("nv_selective_scan: no kernel for %d lanes x %d states", L, SPL);
     return NV_ERR_UNSUPPORTED;
 }
 
@@ -388,7 +430,7 @@ extern "C" int nv_selective_scan(const void* x, int64_t x_stride, const void* dt
     NV_REQUIRE(N <= 256, NV_ERR_UNSUPPORTED, "nv_selective_scan: %d states per channel exceed 256", N);
     NV_REQUIRE(dtype == NV_DTYPE_BF16 || dtype == NV_DTYPE_F32, NV_ERR_INVALID_ARG, "nv_selective_scan: bad dtype");
     const ScPlan p = sc_plan(num_seqs, C, N, max_seqlen_q);
-    NV_REQUIRE((C + kScThreads / p.L - 1) / (kScThreads / p.L) < 65536, NV_ERR_UNSUPPORTED, "nv_selective_scan: launch too large");
+    NV_REQUIRE(C / 4 < 65535, NV_ERR_UNSUPPORTED, "nv_selective_scan: launch too large");
     NV_REQUIRE(p.ws_floats == 0 || (workspace && workspace_bytes >= p.ws_floats * (int64_t)sizeof(float)), NV_ERR_WORKSPACE,
                "nv_selective_scan: workspace of %lld bytes, need %lld", (long long)workspace_bytes,
                (long long)(p.ws_floats * (int64_t)sizeof(float)));
@@ -396,16 +438,17 @@ extern "C" int nv_selective_scan(const void* x, int64_t x_stride, const void* dt
     float* seg_state = (float*)workspace;
     float* seg_dt = p.nseg > 1 ? seg_state + (int64_t)num_seqs * p.nseg * C * N : nullptr;
     const int align = dtype == NV_DTYPE_BF16 ? 8 : 16;
-    const int vec = C % 4 == 0 && x_stride % 4 == 0 && dt_stride % 4 == 0 && z_stride % 4 == 0 && out_stride % 4 == 0 &&
-                    ((uintptr_t)x | (uintptr_t)dt_raw | (uintptr_t)z | (uintptr_t)out) % align == 0;
+    const bool vec = C % 4 == 0 && x_stride % 4 == 0 && dt_stride % 4 == 0 && z_stride % 4 == 0 && out_stride % 4 == 0 &&
+                     N % 4 == 0 && b_stride % 4 == 0 && c_stride % 4 == 0 &&
+                     ((uintptr_t)x | (uintptr_t)dt_raw | (uintptr_t)z | (uintptr_t)out | (uintptr_t)Bm | (uintptr_t)Cm) % align == 0;
     if (dtype == NV_DTYPE_BF16) {
         const ScArgs<__bf16> a{(const __bf16*)x, (const __bf16*)dt_raw, (const __bf16*)z, (const __bf16*)Bm, (const __bf16*)Cm,
                                x_stride, dt_stride, z_stride, b_stride, c_stride, dt_bias, A, D_skip, state, (__bf16*)out,
-                               out_stride, cu_seqlens_q, cu_seqlens_k, state_slots, C, N, p.seg_len, p.nseg, seg_state, seg_dt, vec};
-        return run_scan<__bf16>(a, p, num_seqs, s);
+                               out_stride, cu_seqlens_q, cu_seqlens_k, state_slots, C, N, p.seg_len, p.nseg, seg_state, seg_dt};
+        return run_scan<__bf16>(a, p, vec, num_seqs, s);
     }
     const ScArgs<float> a{(const float*)x, (const float*)dt_raw, (const float*)z, (const float*)Bm, (const float*)Cm, x_stride,
                           dt_stride, z_stride, b_stride, c_stride, dt_bias, A, D_skip, state, (float*)out, out_stride,
-                          cu_seqlens_q, cu_seqlens_k, state_slots, C, N, p.seg_len, p.nseg, seg_state, seg_dt, vec};
-    return run_scan<float>(a, p, num_seqs, s);
+                          cu_seqlens_q, cu_seqlens_k, state_slots, C, N, p.seg_len, p.nseg, seg_state, seg_dt};
+    return run_scan<float>(a, p, vec, num_seqs, s);
 }
