@@ -343,7 +343,7 @@ static ScPlan sc_plan(int B, int C, int N, int max_seqlen_q) {
         p.SPL = 8;
         p.L /= 2;
     }
-    const int64_t waves = (int64_t)B * C * p.L / 64;
+    const int64_t waves = ((int64_t)B * C * p.L + 63) / 64;
     const int mq = std::max(1, max_seqlen_q);
     p.seg_len = (mq + kScTile - 1) / kScTile * kScTile;
     if (waves < 2048 && mq >= 256) {

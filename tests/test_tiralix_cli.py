@@ -119,3 +119,16 @@ def test_generate_program_matches_the_oracle_greedy(tmp_path):
     for _ in range(6):
         seq.append(int(oracle_logits(CFG, ck, seq)[-1].argmax()))
     assert out["token_ids"] == seq[len(prompt):]
+
+
+def test_launch_plans_of_any_size_are_answered():
+    """The workspace queries plan a launch on the host: few channels, long portions, many sequences and one."""
+    from nanovllm_amd import _lib
+    dll = _lib.mixers()
+    for B in (1, 2, 70, 300):
+        for mq in (1, 2, 16, 17, 255, 256, 512, 1000, 100000):
+            for C, N in ((1, 1), (7, 3), (24, 6), (100, 256), (20000, 16)):
+                assert 0 <= dll.nv_selective_scan_workspace_bytes(B, C, N, mq) <= 4 * B * 16 * C * (N + 1)
+            for H, Dk, Dv in ((1, 1, 1), (3, 5, 65), (64, 128, 256)):
+                assert 0 <= dll.nv_fixed_decay_workspace_bytes(B, H, Dk, Dv, mq, 0) <= 4 * B * 16 * H * Dk * Dv
+                assert dll.nv_fixed_decay_workspace_bytes(B, H, Dk, Dv, mq, 1) == 0        # float32 rows run token by token
