@@ -460,35 +460,38 @@ NV_API int nv_attn_latent_paged(const void* q, const void* cache, void* out, con
  *   dt = softplus(dt_raw + dt_bias);  S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n;  y_c = sum_n S[c, n] C_n + D_c x_c
  *   out_c = y_c * silu(z_c)
  * x, dt_raw, z, out: [T, C], Bm, Cm: [T, N] of dtype with row strides; dt_bias, D: [C], A: [C, N] fp32 (A is negative).
- * N <= 256.  max_seqlen_q: the most rows a sequence has in the step; a step with few sequences is cut into segments along
- * time through a workspace of nv_selective_scan_workspace_bytes.
+ * N <= 256.  T: the step's rows, max_seqlen_q: the most rows a sequence has of them, leading_singles: so many sequences lead the
+ * batch with exactly one row each (they get a launch of their own; 0 is always right).  Long portions of few sequences are
+ * cut into segments along time through a workspace of nv_selective_scan_workspace_bytes.
  */
-NV_API int64_t nv_selective_scan_workspace_bytes(int num_seqs, int C, int N, int max_seqlen_q);
+NV_API int64_t nv_selective_scan_workspace_bytes(int num_seqs, int64_t T, int C, int N, int max_seqlen_q, int leading_singles);
 NV_API int nv_selective_scan(const void* x, int64_t x_stride, const void* dt_raw, int64_t dt_stride, const void* z,
                              int64_t z_stride, const void* Bm, int64_t b_stride, const void* Cm, int64_t c_stride,
                              const float* dt_bias, const float* A, const float* D, float* state, void* out,
                              int64_t out_stride, const int32_t* cu_seqlens_q, const int32_t* cu_seqlens_k,
-                             const int32_t* state_slots, int num_seqs, int C, int N, int max_seqlen_q, int dtype,
-                             void* workspace, int64_t workspace_bytes, void* stream);
+                             const int32_t* state_slots, int num_seqs, int64_t T, int C, int N, int max_seqlen_q,
+                             int leading_singles, int dtype, void* workspace, int64_t workspace_bytes, void* stream);
 
 /*
  * Linear attention with one constant decay per head, state [num_slots, H, Dk, Dv] fp32 carried per sequence:
  *   S <- decay_h S + silu(k) silu(v)^T;  o = S^T silu(q)              (out: [T, H * Dv] fp32 with a row stride)
- * q, k: [T, H * Dk]; v: [T, H * Dv] of dtype with row strides; decay: [H] fp32.  Dk, Dv <= 256.  max_seqlen_q: the most rows
- * a sequence has in the step; `portions`: which kinds of portions the step may hold, NV_PORTION_* added up (7: anything; a
- * kind left out is not run).  Single tokens stream the state, portions of at most NV_FEW_ROWS tokens run token by token, longer
- * ones of bf16 rows with Dk <= 128 in chunks on the matrix cores, through a workspace when a step with few sequences is cut
- * into segments along time.
+ * q, k: [T, H * Dk]; v: [T, H * Dv] of dtype with row strides; decay: [H] fp32.  Dk, Dv <= 256.  T, max_seqlen_q, leading_singles
+ * as above; `portions`: which kinds of portions stand behind the leading single tokens, NV_PORTION_* added up (7: anything; a
+ * kind left out is not run).  Leading single tokens stream the state, portions of at most NV_FEW_ROWS tokens run token by
+ * token, longer ones of bf16 rows with Dk <= 128 in chunks on the matrix cores, through a workspace when long portions of few
+ * sequences are cut into segments along time.
  */
 #define NV_FEW_ROWS 16
 #define NV_PORTION_SINGLE 1
-#define NV_PORTION_FEW 2
+#define NV_PORTION_FEW 2        /* 2 .. NV_FEW_ROWS tokens */
 #define NV_PORTION_LONG 4
-NV_API int64_t nv_fixed_decay_workspace_bytes(int num_seqs, int H, int Dk, int Dv, int max_seqlen_q, int dtype);
+NV_API int64_t nv_fixed_decay_workspace_bytes(int num_seqs, int64_t T, int H, int Dk, int Dv, int max_seqlen_q,
+                                              int leading_singles, int dtype);
 NV_API int nv_fixed_decay_memory(const void* q, const void* k, const void* v, int64_t q_stride, int64_t k_stride,
                                  int64_t v_stride, const float* decay, float* state, float* out, int64_t out_stride,
                                  const int32_t* cu_seqlens_q, const int32_t* cu_seqlens_k, const int32_t* state_slots,
-                                 int num_seqs, int H, int Dk, int Dv, int max_seqlen_q, int portions, int dtype,
+                                 int num_seqs, int64_t T, int H, int Dk, int Dv, int max_seqlen_q, int leading_singles,
+                                 int portions, int dtype,
                                  void* workspace, int64_t workspace_bytes, void* stream);
 
 /*

@@ -139,12 +139,12 @@ MIXERS_PROTOTYPES = {
     "nv_attn_latent_workspace_bytes": (_i64, [_i32, _i64, _i32, _i32, _i32, _i32, _i32]),
     "nv_attn_latent_paged": (_i32, [_vp, _vp, _vp, _vp, _vp, _vp, _i32, _i32, _i64, _i32, _i32, _i32, _i64, _i32, _f32, _vp, _i32,
                                     _i32, _i32, _vp, _i64, _vp]),
-    "nv_selective_scan_workspace_bytes": (_i64, [_i32, _i32, _i32, _i32]),
+    "nv_selective_scan_workspace_bytes": (_i64, [_i32, _i64, _i32, _i32, _i32, _i32]),
     "nv_selective_scan": (_i32, [_vp, _i64, _vp, _i64, _vp, _i64, _vp, _i64, _vp, _i64, _vp, _vp, _vp, _vp, _vp, _i64, _vp, _vp,
-                                 _vp, _i32, _i32, _i32, _i32, _i32, _vp, _i64, _vp]),
-    "nv_fixed_decay_workspace_bytes": (_i64, [_i32, _i32, _i32, _i32, _i32, _i32]),
-    "nv_fixed_decay_memory": (_i32, [_vp, _vp, _vp, _i64, _i64, _i64, _vp, _vp, _vp, _i64, _vp, _vp, _vp, _i32, _i32, _i32, _i32,
-                                     _i32, _i32, _i32, _vp, _i64, _vp]),
+                                 _vp, _i32, _i64, _i32, _i32, _i32, _i32, _i32, _vp, _i64, _vp]),
+    "nv_fixed_decay_workspace_bytes": (_i64, [_i32, _i64, _i32, _i32, _i32, _i32, _i32, _i32]),
+    "nv_fixed_decay_memory": (_i32, [_vp, _vp, _vp, _i64, _i64, _i64, _vp, _vp, _vp, _i64, _vp, _vp, _vp, _i32, _i64, _i32, _i32,
+                                     _i32, _i32, _i32, _i32, _i32, _vp, _i64, _vp]),
     "nv_row_norm_rope_store": (_i32, [_vp, _vp, _vp, _i64, _i64, _i64, _vp, _vp, _f32, _vp, _i32, _f32, _vp, _vp, _vp, _vp, _vp,
                                       _i32, _i64, _i32, _i32, _i32, _i32, _vp]),
     "nv_join_gated": (_i32, [_vp, _i64, _vp, _i64, _i32, _i32, _f32, _vp, _i64, _vp, _vp, _i64, _i32, _f32, _f32, _vp, _i32, _i64,

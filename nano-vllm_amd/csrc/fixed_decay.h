@@ -16,8 +16,7 @@ struct FixedDecayArgs {
     int num_seqs, H, Dk, Dv;
 };
 
-// Token by token with the state in registers, every sequence with min_rows .. max_rows rows in the step; any sizes up to
-// 256 x 256.
-int launch_fixed_decay_rows(const FixedDecayArgs& f, int dtype, int min_rows, int max_rows, hipStream_t s);
+// Token by token with the state in registers, every sequence with at most max_rows rows in the step; any sizes up to 256 x 256.
+int launch_fixed_decay_rows(const FixedDecayArgs& f, int dtype, int max_rows, hipStream_t s);
 
 }  // namespace nv

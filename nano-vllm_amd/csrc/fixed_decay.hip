@@ -20,13 +20,14 @@
 // holds rows 4 g .. 4 g + 3 of two stacked 16-row tiles (g: its group of 16 lanes), so the contraction index runs in the
 // order 16 (e / 4) + 4 g + e % 4, and the other operand is read in the same order (two 8-byte reads, or two transposed ones).
 //
-// Long sequences in a step that does not fill the chip are cut into segments as in selective_scan.hip; the decay of a whole
-// segment is decay^length.
+// Long portions in a step that does not fill the chip are cut into segments (segments.h); the decay of a whole segment is
+// decay^length.
 #include <algorithm>
 
 #include "fixed_decay.h"
 #include "mfma_tile.h"
 #include "row_pieces.h"
+#include "segments.h"
 #include "../../include/nanovllm_hip_mixers.h"
 
 namespace nv {
@@ -40,7 +41,7 @@ constexpr int kFdVs = 64 + 8;                  // LDS row of the values, in elem
 struct FdParams {
     FixedDecayArgs f;
     int seg_len, nseg;                         // tokens per segment (a multiple of kFdChunk)
-    float* seg_state;                          // [B, nseg, H, Dk, Dv]
+    float* seg_state;                          // [places, H, Dk, Dv]
 };
 
 __device__ __forceinline__ float fd_silu(float x) {
@@ -105,7 +106,7 @@ __global__ __launch_bounds__(256) void fixed_decay_chunk_kernel(const FdParams p
     const int b = blockIdx.x, h = blockIdx.y % H, cg = blockIdx.y / H, seg = blockIdx.z;
     const int q0 = f.cu_q[b], len_q = f.cu_q[b + 1] - q0;
     if (len_q <= kFdFewRows) return;
-    const int first = seg * p.seg_len, last_seg = min((len_q - 1) / p.seg_len, p.nseg - 1);
+    const int first = seg * p.seg_len, last_seg = segment_count(len_q, p.seg_len, p.nseg) - 1;
     if (seg > last_seg) return;
     const int start = (f.cu_k[b + 1] - f.cu_k[b]) - len_q;
     const int tid = threadIdx.x, lane = tid & 63, l15 = lane & 15, g = lane >> 4;
@@ -113,7 +114,9 @@ __global__ __launch_bounds__(256) void fixed_decay_chunk_kernel(const FdParams p
     const int col = cg * 64 + wave * 16 + l15;                   // the lane's value column of the state
     const float decay = f.decay[h];
     float* slot_state = f.state + ((int64_t)f.slots[b] * H + h) * (int64_t)Dk * Dv;
-    auto seg_at = [&](int s) { return p.seg_state + (((int64_t)b * p.nseg + s) * H + h) * (int64_t)Dk * Dv; };
+    int64_t place = 0;                                           // of the sequence's first segment
+    if (MODE != kFdWhole && last_seg > 0) place = segment_first_place(f.cu_q, b, p.seg_len, p.nseg);
+    auto seg_at = [&](int s) { return p.seg_state + ((place + s) * H + h) * (int64_t)Dk * Dv; };
 
     f32x4 S[2 * DKT];                                            // S[t][r]: key channel 16 t + 4 g + r, value column col
 #pragma unroll
@@ -395,18 +398,21 @@ static bool fd_chunked(int Dk, int Dv, int dtype, int max_seqlen_q) {
     return dtype == NV_DTYPE_BF16 && Dk <= 128 && Dv <= 256 && max_seqlen_q > kFdFewRows;
 }
 
-// Segments so that the launch has about two workgroups per CU.
-static FdPlan fd_plan(int B, int H, int Dk, int Dv, int max_seqlen_q) {
+// Segments so that the launch has about two workgroups per CU.  The sequences that count are the long ones: T rows make at most
+// that many portions of the longest one's length.
+static FdPlan fd_plan(int B, int64_t T, int H, int Dk, int Dv, int max_seqlen_q, int lead) {
+    B -= lead;
+    T -= lead;
     const int mq = std::max(1, max_seqlen_q);
     FdPlan p{1, (mq + kFdChunk - 1) / kFdChunk * kFdChunk, 0};
-    const int64_t groups = (int64_t)B * H * ((Dv + 63) / 64);
-    if (groups < 256 && mq >= 512) {
+    const int64_t groups = std::max<int64_t>(1, std::min<int64_t>(B, (T + mq - 1) / mq)) * H * ((Dv + 63) / 64);
+    if (B > 0 && groups < 256 && mq >= 512) {
         const int want = (int)std::min<int64_t>((512 + groups - 1) / groups, 16);
         p.nseg = std::max(1, std::min(want, mq / 256));
         p.seg_len = ((mq + p.nseg - 1) / p.nseg + kFdChunk - 1) / kFdChunk * kFdChunk;
         p.nseg = (mq + p.seg_len - 1) / p.seg_len;
     }
-    if (p.nseg > 1) p.ws_floats = (int64_t)B * p.nseg * H * Dk * Dv;
+    if (p.nseg > 1) p.ws_floats = segment_places(T, p.seg_len) * H * Dk * Dv;
     return p;
 }
 
@@ -427,20 +433,24 @@ static void launch_chunks(const FdParams& p, bool vec, hipStream_t s) {
 
 }  // namespace nv
 
-extern "C" int64_t nv_fixed_decay_workspace_bytes(int num_seqs, int H, int Dk, int Dv, int max_seqlen_q, int dtype) {
-    if (num_seqs <= 0 || H <= 0 || Dk <= 0 || Dv <= 0 || !nv::fd_chunked(Dk, Dv, dtype, max_seqlen_q)) return 0;
-    return nv::fd_plan(num_seqs, H, Dk, Dv, max_seqlen_q).ws_floats * (int64_t)sizeof(float);
+extern "C" int64_t nv_fixed_decay_workspace_bytes(int num_seqs, int64_t T, int H, int Dk, int Dv, int max_seqlen_q,
+                                                  int leading_singles, int dtype) {
+    if (num_seqs <= 0 || T <= 0 || leading_singles < 0 || leading_singles > num_seqs || H <= 0 || Dk <= 0 || Dv <= 0 || !nv::fd_chunked(Dk, Dv, dtype, max_seqlen_q)) return 0;
+    return nv::fd_plan(num_seqs, T, H, Dk, Dv, max_seqlen_q, leading_singles).ws_floats * (int64_t)sizeof(float);
 }
 
 extern "C" int nv_fixed_decay_memory(const void* q, const void* k, const void* v, int64_t q_stride, int64_t k_stride,
                                      int64_t v_stride, const float* decay, float* state, float* out, int64_t out_stride,
                                      const int32_t* cu_seqlens_q, const int32_t* cu_seqlens_k, const int32_t* state_slots,
-                                     int num_seqs, int H, int Dk, int Dv, int max_seqlen_q, int portions, int dtype,
+                                     int num_seqs, int64_t T, int H, int Dk, int Dv, int max_seqlen_q, int leading_singles,
+                                     int portions, int dtype,
                                      void* workspace, int64_t workspace_bytes, void* stream) {
     using namespace nv;
-    NV_REQUIRE(num_seqs >= 0 && H > 0 && Dk > 0 && Dv > 0 && max_seqlen_q >= 1, NV_ERR_INVALID_ARG,
+    NV_REQUIRE(num_seqs >= 0 && T >= 0 && H > 0 && Dk > 0 && Dv > 0 && max_seqlen_q >= 1 && leading_singles >= 0 &&
+                   leading_singles <= num_seqs,
+               NV_ERR_INVALID_ARG,
                "nv_fixed_decay_memory: bad sizes");
-    if (num_seqs == 0) return NV_OK;
+    if (num_seqs == 0 || T == 0) return NV_OK;
     NV_REQUIRE(q && k && v && decay && state && out && cu_seqlens_q && cu_seqlens_k && state_slots, NV_ERR_INVALID_ARG,
                "nv_fixed_decay_memory: null pointer");
     NV_REQUIRE(Dk <= 256 && Dv <= 256, NV_ERR_UNSUPPORTED, "nv_fixed_decay_memory: Dk=%d, Dv=%d exceed 256", Dk, Dv);
@@ -450,21 +460,25 @@ extern "C" int nv_fixed_decay_memory(const void* q, const void* k, const void* v
     FdParams p{};
     p.f = FixedDecayArgs{q,          k,          v,          q_stride, k_stride, v_stride, decay, state, out,
                          out_stride, cu_seqlens_q, cu_seqlens_k, state_slots, num_seqs, H,        Dk,       Dv};
-    // the launches a sequence of this many rows belongs to
     const bool chunked = fd_chunked(Dk, Dv, dtype, max_seqlen_q);
-    if (portions & NV_PORTION_SINGLE) {
+    if (leading_singles > 0) {
         NV_REQUIRE((uintptr_t)state % 16 == 0, NV_ERR_INVALID_ARG, "nv_fixed_decay_memory: the state must start on 16 bytes");
+        p.f.num_seqs = leading_singles;
         if (dtype == NV_DTYPE_BF16) launch_single<__bf16>(p.f, s);
         else launch_single<float>(p.f, s);
         const int rc = check_launch("nv_fixed_decay_memory (single tokens)");
-        if (rc != NV_OK) return rc;
+        if (rc != NV_OK || leading_singles == num_seqs) return rc;
+        p.f.num_seqs = num_seqs - leading_singles;               // (row numbers stay those of the step)
+        p.f.cu_q += leading_singles;
+        p.f.cu_k += leading_singles;
+        p.f.slots += leading_singles;
     }
-    if ((portions & NV_PORTION_FEW) || (!chunked && (portions & NV_PORTION_LONG))) {
-        const int rc = launch_fixed_decay_rows(p.f, dtype, 2, chunked ? kFdFewRows : 1 << 30, s);
+    if ((portions & (NV_PORTION_SINGLE | NV_PORTION_FEW)) || (!chunked && (portions & NV_PORTION_LONG))) {
+        const int rc = launch_fixed_decay_rows(p.f, dtype, chunked ? kFdFewRows : 1 << 30, s);
         if (rc != NV_OK) return rc;
     }
     if (!chunked || !(portions & NV_PORTION_LONG)) return NV_OK;
-    const FdPlan plan = fd_plan(num_seqs, H, Dk, Dv, max_seqlen_q);
+    const FdPlan plan = fd_plan(num_seqs, T, H, Dk, Dv, max_seqlen_q, leading_singles);
     NV_REQUIRE(plan.ws_floats == 0 || (workspace && workspace_bytes >= plan.ws_floats * (int64_t)sizeof(float)), NV_ERR_WORKSPACE,
                "nv_fixed_decay_memory: workspace of %lld bytes, need %lld", (long long)workspace_bytes,
                (long long)(plan.ws_floats * (int64_t)sizeof(float)));

@@ -68,7 +68,7 @@ struct GmArgs {
     int tile;
     const float* decay;                    // fixed form: [H]
     float* out32;                          // fixed form: [T, H * Dv]
-    int min_rows, max_rows;                // fixed form: sequences with other numbers of rows belong to other launches
+    int max_rows;                          // fixed form: sequences with more rows belong to another launch
 };
 
 template <typename T, int RPL, int FORM, int MAXT>
@@ -91,7 +91,7 @@ __global__ __launch_bounds__(MAXT) void gated_memory_kernel(const GmArgs<T> a) {
     const int q0 = a.cu_q[b], len_q = a.cu_q[b + 1] - q0;
     if (len_q <= 0) return;
     if constexpr (FORM == kGmFixed)
-        if (len_q < a.min_rows || len_q > a.max_rows) return;
+        if (len_q > a.max_rows) return;
     const int start = (a.cu_k[b + 1] - a.cu_k[b]) - len_q;
     const int col = wave * 16 + (lane >> 2), q = lane & 3;
     const bool live = col < Dv;
@@ -284,7 +284,7 @@ static int launch_gated_memory(GmArgs<T> a, int B, hipStream_t s, const char* wh
     return check_launch(what);
 }
 
-int launch_fixed_decay_rows(const FixedDecayArgs& f, int dtype, int min_rows, int max_rows, hipStream_t s) {
+int launch_fixed_decay_rows(const FixedDecayArgs& f, int dtype, int max_rows, hipStream_t s) {
     auto fill = [&](auto* none) {
         using T = std::remove_pointer_t<decltype(none)>;
         GmArgs<T> a{};
@@ -304,7 +304,6 @@ int launch_fixed_decay_rows(const FixedDecayArgs& f, int dtype, int min_rows, in
         a.Dv = f.Dv;
         a.decay = f.decay;
         a.out32 = f.out;
-        a.min_rows = min_rows;
         a.max_rows = max_rows;
         return launch_gated_memory<T, kGmFixed>(a, f.num_seqs, s, "nv_fixed_decay_memory");
     };
@@ -335,13 +334,13 @@ extern "C" int nv_mlstm_memory(const void* q, const void* k, const void* v, int6
         GmArgs<__bf16> a{(const __bf16*)q, (const __bf16*)k, (const __bf16*)v, q_stride, k_stride, v_stride, nullptr, 0,
                          i_pre, f_pre, gate_pre_stride, (const __bf16*)gate_raw, gate_stride, i_bias, f_bias, nullptr,
                          norm_w, Dv, state, norm_state, max_state, (__bf16*)out, out_stride, cu_seqlens_q, cu_seqlens_k,
-                         state_slots, H, Dk, Dv, eps, gate_cap, q_scale, 0, nullptr, nullptr, 0, 0};
+                         state_slots, H, Dk, Dv, eps, gate_cap, q_scale, 0, nullptr, nullptr, 0};
         return launch_gated_memory<__bf16, kGmMatrix>(a, num_seqs, s, "nv_mlstm_memory");
     }
     GmArgs<float> a{(const float*)q, (const float*)k, (const float*)v, q_stride, k_stride, v_stride, nullptr, 0, i_pre,
                     f_pre, gate_pre_stride, (const float*)gate_raw, gate_stride, i_bias, f_bias, nullptr, norm_w, Dv,
                     state, norm_state, max_state, (float*)out, out_stride, cu_seqlens_q, cu_seqlens_k, state_slots, H, Dk,
-                    Dv, eps, gate_cap, q_scale, 0, nullptr, nullptr, 0, 0};
+                    Dv, eps, gate_cap, q_scale, 0, nullptr, nullptr, 0};
     return launch_gated_memory<float, kGmMatrix>(a, num_seqs, s, "nv_mlstm_memory");
 }
 
@@ -362,11 +361,11 @@ extern "C" int nv_gated_write_memory(const void* q, const void* f_raw, const voi
     if (dtype == NV_DTYPE_BF16) {
         GmArgs<__bf16> a{(const __bf16*)q, nullptr, (const __bf16*)v, q_stride, 0, v_stride, (const __bf16*)f_raw, f_stride,
                          nullptr, nullptr, 0, nullptr, 0, nullptr, f_bias, lower, norm_w, 0, state, nullptr, nullptr,
-                         (__bf16*)out, out_stride, cu_seqlens_q, cu_seqlens_k, state_slots, H, Dk, Dv, eps, 0.f, 1.f, 0, nullptr, nullptr, 0, 0};
+                         (__bf16*)out, out_stride, cu_seqlens_q, cu_seqlens_k, state_slots, H, Dk, Dv, eps, 0.f, 1.f, 0, nullptr, nullptr, 0};
         return launch_gated_memory<__bf16, kGmWrite>(a, num_seqs, s, "nv_gated_write_memory");
     }
     GmArgs<float> a{(const float*)q, nullptr, (const float*)v, q_stride, 0, v_stride, (const float*)f_raw, f_stride, nullptr,
                     nullptr, 0, nullptr, 0, nullptr, f_bias, lower, norm_w, 0, state, nullptr, nullptr, (float*)out,
-                    out_stride, cu_seqlens_q, cu_seqlens_k, state_slots, H, Dk, Dv, eps, 0.f, 1.f, 0, nullptr, nullptr, 0, 0};
+                    out_stride, cu_seqlens_q, cu_seqlens_k, state_slots, H, Dk, Dv, eps, 0.f, 1.f, 0, nullptr, nullptr, 0};
     return launch_gated_memory<float, kGmWrite>(a, num_seqs, s, "nv_gated_write_memory");
 }

@@ -13,13 +13,13 @@
 // C once per token), the next 16 tokens' inputs being on their way into registers meanwhile; the token loop has no
 // barrier: two small LDS reads per vector, one exponential and three multiply-adds per state, a sum over the L lanes.
 //
-// A step with too few (sequence, channel) pairs to fill the chip is cut into segments along time: a first launch runs every
-// segment but a sequence's last from a zero state and leaves its end state and its sum of dt per channel (the decay of a
-// whole segment is exp(A * sum dt)); in the second launch a segment folds what is in front of it into its start state and
-// runs as usual.
+// A step with too few (sequence, channel) pairs to fill the chip is cut into segments along time (segments.h); what a segment
+// leaves is its end state and its sum of dt per channel: the decay of a whole segment is exp(A * sum dt).  Leading single
+// tokens have a launch of their own.
 #include <algorithm>
 
 #include "row_pieces.h"
+#include "segments.h"
 #include "../../include/nanovllm_hip_mixers.h"
 
 namespace nv {
@@ -94,7 +94,7 @@ struct ScArgs {
     const int *cu_q, *cu_k, *slots;
     int C, N;
     int seg_len, nseg;                         // tokens per segment (a multiple of kScTile), segments of the longest sequence
-    float *seg_state, *seg_dt;                 // [B, nseg, C, N], [B, nseg, C]
+    float *seg_state, *seg_dt;                 // [places, C, N], [places, C]
 };
 
 // Four neighbouring columns of a row as they lie in memory (zeros from `cols` on): what is on its way must not be touched.
@@ -139,7 +139,7 @@ __global__ __launch_bounds__(kScThreads) void selective_scan_kernel(const ScArgs
     const int b = blockIdx.x, c0 = blockIdx.y * CPB, seg = blockIdx.z;
     const int q0 = a.cu_q[b], len_q = a.cu_q[b + 1] - q0;
     if (len_q <= 0) return;
-    const int first = seg * a.seg_len, last_seg = min((len_q - 1) / a.seg_len, a.nseg - 1);
+    const int first = seg * a.seg_len, last_seg = segment_count(len_q, a.seg_len, a.nseg) - 1;
     if (seg > last_seg) return;
     const int start = (a.cu_k[b + 1] - a.cu_k[b]) - len_q;
     const int tid = threadIdx.x, ch = tid / L, sub = tid % L;
@@ -154,19 +154,21 @@ __global__ __launch_bounds__(kScThreads) void selective_scan_kernel(const ScArgs
         A2[i] *= kScLog2e;
         S[i] = 0.f;
     }
+    int64_t place = 0;                                           // of the sequence's first segment
+    if (MODE != kScWhole && last_seg > 0) place = segment_first_place(a.cu_q, b, a.seg_len, a.nseg);
     if constexpr (MODE == kScSummary) {
         if (last_seg == 0) return;                               // nobody folds
         if (seg == last_seg) {                                   // the start state is handed on from here: the second launch
             if (!live) return;                                   // overwrites the slot
             sc_load_states<SPL>(slot_state, n0, N, start > 0, S);
-            sc_store_states<SPL>(a.seg_state + (((int64_t)b * a.nseg + seg) * C + c) * N, n0, N, S);
+            sc_store_states<SPL>(a.seg_state + ((place + seg) * C + c) * N, n0, N, S);
             return;
         }
     } else {
         if (MODE == kScFinal && last_seg > 0) {
-            sc_load_states<SPL>(a.seg_state + (((int64_t)b * a.nseg + last_seg) * C + c) * N, n0, N, live, S);
+            sc_load_states<SPL>(a.seg_state + ((place + last_seg) * C + c) * N, n0, N, live, S);
             for (int s = 0; s < seg; ++s) {
-                const int64_t at = ((int64_t)b * a.nseg + s) * C + c;
+                const int64_t at = (place + s) * C + c;
                 const float dsum = live ? a.seg_dt[at] : 0.f;
                 float loc[SPL];
                 sc_load_states<SPL>(a.seg_state + at * N, n0, N, live, loc);
@@ -285,7 +287,7 @@ __global__ __launch_bounds__(kScThreads) void selective_scan_kernel(const ScArgs
     }
     if (!live) return;
     if constexpr (MODE == kScSummary) {
-        const int64_t at = ((int64_t)b * a.nseg + seg) * C + c;
+        const int64_t at = (place + seg) * C + c;
         if (sub == 0) a.seg_dt[at] = dt_sum;
         sc_store_states<SPL>(a.seg_state + at * N, n0, N, S);
     } else if (seg == last_seg) {
@@ -330,30 +332,29 @@ struct ScPlan {
     int64_t ws_floats;
 };
 
-// Lanes per channel and states per lane from N; segments so that the launch has about two waves per SIMD.
-static ScPlan sc_plan(int B, int C, int N, int max_seqlen_q) {
+// Lanes per channel and states per lane from N; segments so that the launch has about four waves per SIMD.  The sequences that
+// count are the long ones: T rows make at most that many portions of the longest one's length.
+static ScPlan sc_plan(int B, int64_t T, int C, int N, int max_seqlen_q, int lead) {
     ScPlan p{1, 4, 1, 0, 0};
+    B -= lead;
+    T -= lead;
     while (p.L * 4 < N) p.L *= 2;
-    if (max_seqlen_q == 1) {
-        p.seg_len = 1;
-        return p;
-    }
+    const int mq = std::max(1, max_seqlen_q);
+    const int64_t seqs = std::max<int64_t>(0, std::min<int64_t>(B, (T + mq - 1) / mq));
     // eight states per lane (half the lanes, less work per token beside the states) when there are plenty of waves
-    if (p.L >= 4 && (int64_t)B * C * p.L / 64 >= 8192) {
+    if (p.L >= 4 && seqs * C * p.L / 64 >= 8192) {
         p.SPL = 8;
         p.L /= 2;
     }
-    const int64_t waves = ((int64_t)B * C * p.L + 63) / 64;
-    const int mq = std::max(1, max_seqlen_q);
+    const int64_t waves = std::max<int64_t>(1, seqs * C * p.L / 64);
     p.seg_len = (mq + kScTile - 1) / kScTile * kScTile;
-    if (waves < 2048 && mq >= 256) {
+    if (seqs > 0 && waves < 2048 && mq >= 256) {
         const int want = (int)std::min<int64_t>((4096 + waves - 1) / waves, 16);
-        const int most = mq / 128;
-        p.nseg = std::max(1, std::min(want, most));
+        p.nseg = std::max(1, std::min(want, mq / 128));
         p.seg_len = ((mq + p.nseg - 1) / p.nseg + kScTile - 1) / kScTile * kScTile;
         p.nseg = (mq + p.seg_len - 1) / p.seg_len;
     }
-    if (p.nseg > 1) p.ws_floats = (int64_t)B * p.nseg * C * (N + 1);
+    if (p.nseg > 1) p.ws_floats = segment_places(T, p.seg_len) * C * (N + 1);
     return p;
 }
 
@@ -370,73 +371,83 @@ static void launch_scan(const ScArgs<T>& a, int B, hipStream_t s) {
 }
 
 template <typename T>
-static int run_scan(ScArgs<T> a, const ScPlan& p, bool vec, int B, hipStream_t s) {
-    int L = p.L, SPL = p.SPL;
-    const bool single = a.seg_len == 1;                          // (max_seqlen_q == 1)
-    if (!single && !vec) {                                       // rows of odd sizes: one plain form
-        L = L * SPL / 4;
-        SPL = 4;
-        a.nseg = 1;
-    }
+static int run_scan(ScArgs<T> a, const ScPlan& p, bool vec, int lead, int B, hipStream_t s) {
+    const int lanes = p.L * p.SPL / 4;                           // at four states per lane
+    if (lead > 0) {
+        bool done = false;
 #define NV_SC_SINGLE(LL)                                                                                                       \
-    if (single && L == LL) {                                                                                                    \
-        constexpr int CPS = kScThreads / LL;                                                                              \
-        hipLaunchKernelGGL((selective_scan_single_kernel<T, LL, 4>), dim3((unsigned)B, (unsigned)((a.C + CPS - 1) / CPS)),       \
-                           dim3(kScThreads), 0, s, a);                                                                    \
+    if (lanes == LL) {                                                                                                          \
+        constexpr int CPS = kScThreads / LL;                                                                                    \
+        hipLaunchKernelGGL((selective_scan_single_kernel<T, LL, 4>), dim3((unsigned)lead, (unsigned)((a.C + CPS - 1) / CPS)),    \
+                           dim3(kScThreads), 0, s, a);                                                                          \
+        done = true;                                                                                                            \
+    }
+        NV_SC_SINGLE(1) NV_SC_SINGLE(2) NV_SC_SINGLE(4) NV_SC_SINGLE(8) NV_SC_SINGLE(16) NV_SC_SINGLE(32) NV_SC_SINGLE(64)
+#undef NV_SC_SINGLE
+        NV_REQUIRE(done, NV_ERR_UNSUPPORTED, "nv_selective_scan: no kernel for %d lanes", lanes);
+        const int rc = check_launch("nv_selective_scan (single tokens)");
+        if (rc != NV_OK || lead == B) return rc;
+        a.cu_q += lead;                                          // (row numbers stay those of the step)
+        a.cu_k += lead;
+        a.slots += lead;
+        B -= lead;
+    }
+    if (!vec) {                                                  // rows of odd sizes: one plain form
+        a.nseg = 1;
+#define NV_SC_PLAIN(LL)                                                                                                        \
+    if (lanes == LL) {                                                                                                          \
+        constexpr int CPB = kScThreads / LL;                                                                                    \
+        hipLaunchKernelGGL((selective_scan_kernel<T, LL, 4, kScWhole, false>), dim3((unsigned)B, (unsigned)((a.C + CPB - 1) / CPB)), \
+                           dim3(kScThreads), 0, s, a);                                                                          \
         return check_launch("nv_selective_scan");                                                                               \
     }
+        NV_SC_PLAIN(1) NV_SC_PLAIN(2) NV_SC_PLAIN(4) NV_SC_PLAIN(8) NV_SC_PLAIN(16) NV_SC_PLAIN(32) NV_SC_PLAIN(64)
+#undef NV_SC_PLAIN
+    }
 #define NV_SC(LL, SS)                                                                                                          \
-    if (!single && vec && L == LL && SPL == SS) {                                                                               \
+    if (p.L == LL && p.SPL == SS) {                                                                                             \
         launch_scan<T, LL, SS>(a, B, s);                                                                                        \
         return check_launch("nv_selective_scan");                                                                               \
     }
-#define NV_SC_PLAIN(LL)                                                                                                        \
-    if (!single && !vec && L == LL) {                                                                                           \
-        constexpr int CPB = kScThreads / LL;                                                                                \
-        hipLaunchKernelGGL((selective_scan_kernel<T, LL, 4, kScWhole, false>), dim3((unsigned)B, (unsigned)((a.C + CPB - 1) / CPB)), \
-                           dim3(kScThreads), 0, s, a);                                                                      \
-        return check_launch("nv_selective_scan");                                                                               \
-    }
-    NV_SC_SINGLE(1) NV_SC_SINGLE(2) NV_SC_SINGLE(4) NV_SC_SINGLE(8) NV_SC_SINGLE(16) NV_SC_SINGLE(32) NV_SC_SINGLE(64)
     NV_SC(1, 4) NV_SC(2, 4) NV_SC(4, 4) NV_SC(8, 4) NV_SC(16, 4) NV_SC(32, 4) NV_SC(64, 4)
     NV_SC(2, 8) NV_SC(4, 8) NV_SC(8, 8) NV_SC(16, 8) NV_SC(32, 8)
-    NV_SC_PLAIN(1) NV_SC_PLAIN(2) NV_SC_PLAIN(4) NV_SC_PLAIN(8) NV_SC_PLAIN(16) NV_SC_PLAIN(32) NV_SC_PLAIN(64)
-#undef NV_SC_SINGLE
 #undef NV_SC
-#undef NV_SC_PLAIN
-    set_error("nv_selective_scan: no kernel for %d lanes x %d states", L, SPL);
+    set_error("nv_selective_scan: no kernel for %d lanes x %d states", p.L, p.SPL);
     return NV_ERR_UNSUPPORTED;
 }
 
 }  // namespace nv
 
-extern "C" int64_t nv_selective_scan_workspace_bytes(int num_seqs, int C, int N, int max_seqlen_q) {
-    if (num_seqs <= 0 || C <= 0 || N <= 0 || N > 256) return 0;
-    return nv::sc_plan(num_seqs, C, N, max_seqlen_q).ws_floats * (int64_t)sizeof(float);
+extern "C" int64_t nv_selective_scan_workspace_bytes(int num_seqs, int64_t T, int C, int N, int max_seqlen_q, int leading_singles) {
+    if (num_seqs <= 0 || T <= 0 || leading_singles < 0 || leading_singles > num_seqs || C <= 0 || N <= 0 || N > 256) return 0;
+    return nv::sc_plan(num_seqs, T, C, N, max_seqlen_q, leading_singles).ws_floats * (int64_t)sizeof(float);
 }
 
 extern "C" int nv_selective_scan(const void* x, int64_t x_stride, const void* dt_raw, int64_t dt_stride, const void* z,
                                  int64_t z_stride, const void* Bm, int64_t b_stride, const void* Cm, int64_t c_stride,
                                  const float* dt_bias, const float* A, const float* D_skip, float* state, void* out,
                                  int64_t out_stride, const int32_t* cu_seqlens_q, const int32_t* cu_seqlens_k,
-                                 const int32_t* state_slots, int num_seqs, int C, int N, int max_seqlen_q, int dtype,
+                                 const int32_t* state_slots, int num_seqs, int64_t T, int C, int N, int max_seqlen_q,
+                                 int leading_singles, int dtype,
                                  void* workspace, int64_t workspace_bytes, void* stream) {
     using namespace nv;
-    NV_REQUIRE(num_seqs >= 0 && C > 0 && N > 0 && max_seqlen_q >= 1, NV_ERR_INVALID_ARG, "nv_selective_scan: bad sizes");
-    if (num_seqs == 0) return NV_OK;
+    NV_REQUIRE(num_seqs >= 0 && T >= 0 && C > 0 && N > 0 && max_seqlen_q >= 1 && leading_singles >= 0 &&
+                   leading_singles <= num_seqs,
+               NV_ERR_INVALID_ARG, "nv_selective_scan: bad sizes");
+    if (num_seqs == 0 || T == 0) return NV_OK;
     NV_REQUIRE(x && dt_raw && z && Bm && Cm && dt_bias && A && D_skip && state && out && cu_seqlens_q && cu_seqlens_k &&
                    state_slots,
                NV_ERR_INVALID_ARG, "nv_selective_scan: null pointer");
     NV_REQUIRE(N <= 256, NV_ERR_UNSUPPORTED, "nv_selective_scan: %d states per channel exceed 256", N);
     NV_REQUIRE(dtype == NV_DTYPE_BF16 || dtype == NV_DTYPE_F32, NV_ERR_INVALID_ARG, "nv_selective_scan: bad dtype");
-    const ScPlan p = sc_plan(num_seqs, C, N, max_seqlen_q);
+    const ScPlan p = sc_plan(num_seqs, T, C, N, max_seqlen_q, leading_singles);
     NV_REQUIRE(C / 4 < 65535, NV_ERR_UNSUPPORTED, "nv_selective_scan: launch too large");
     NV_REQUIRE(p.ws_floats == 0 || (workspace && workspace_bytes >= p.ws_floats * (int64_t)sizeof(float)), NV_ERR_WORKSPACE,
                "nv_selective_scan: workspace of %lld bytes, need %lld", (long long)workspace_bytes,
                (long long)(p.ws_floats * (int64_t)sizeof(float)));
     hipStream_t s = (hipStream_t)stream;
     float* seg_state = (float*)workspace;
-    float* seg_dt = p.nseg > 1 ? seg_state + (int64_t)num_seqs * p.nseg * C * N : nullptr;
+    float* seg_dt = p.nseg > 1 ? seg_state + segment_places(T - leading_singles, p.seg_len) * C * N : nullptr;
     const int align = dtype == NV_DTYPE_BF16 ? 8 : 16;
     const bool vec = C % 4 == 0 && x_stride % 4 == 0 && dt_stride % 4 == 0 && z_stride % 4 == 0 && out_stride % 4 == 0 &&
                      N % 4 == 0 && b_stride % 4 == 0 && c_stride % 4 == 0 &&
@@ -445,10 +456,10 @@ extern "C" int nv_selective_scan(const void* x, int64_t x_stride, const void* dt
         const ScArgs<__bf16> a{(const __bf16*)x, (const __bf16*)dt_raw, (const __bf16*)z, (const __bf16*)Bm, (const __bf16*)Cm,
                                x_stride, dt_stride, z_stride, b_stride, c_stride, dt_bias, A, D_skip, state, (__bf16*)out,
                                out_stride, cu_seqlens_q, cu_seqlens_k, state_slots, C, N, p.seg_len, p.nseg, seg_state, seg_dt};
-        return run_scan<__bf16>(a, p, vec, num_seqs, s);
+        return run_scan<__bf16>(a, p, vec, leading_singles, num_seqs, s);
     }
     const ScArgs<float> a{(const float*)x, (const float*)dt_raw, (const float*)z, (const float*)Bm, (const float*)Cm, x_stride,
                           dt_stride, z_stride, b_stride, c_stride, dt_bias, A, D_skip, state, (float*)out, out_stride,
                           cu_seqlens_q, cu_seqlens_k, state_slots, C, N, p.seg_len, p.nseg, seg_state, seg_dt};
-    return run_scan<float>(a, p, vec, num_seqs, s);
+    return run_scan<float>(a, p, vec, leading_singles, num_seqs, s);
 }

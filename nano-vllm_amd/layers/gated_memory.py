@@ -79,4 +79,4 @@ class FixedDecayMemory(nn.Module):
         """q, k: [T, H, Dk]; v: [T, H, Dv] as projected; returns [T, H * Dv] float32."""
         ctx = get_context()
         return ops.fixed_decay_memory(q, k, v, self.decay, cache["state"], ctx.cu_seqlens_q, ctx.cu_seqlens_k, ctx.state_slots,
-                                      ctx.max_seqlen_q, ctx.portion_kinds)
+                                      ctx.max_seqlen_q, ctx.num_leading_decode or 0, ctx.portion_kinds)

@@ -106,4 +106,4 @@ class SelectiveScan(nn.Module):
         x's dtype, [T, channels]."""
         ctx = get_context()
         return ops.selective_scan(x, dt_raw, z, B, C, self.dt_bias, self.A, self.D, state, ctx.cu_seqlens_q, ctx.cu_seqlens_k,
-                                  ctx.state_slots, ctx.max_seqlen_q)
+                                  ctx.state_slots, ctx.max_seqlen_q, ctx.num_leading_decode or 0)

@@ -1551,11 +1551,23 @@ def moe_route_softmax(logits: torch.Tensor, correction: Optional[torch.Tensor], 
 # Two mixers side by side on one input (softmax attention with whole-row norms and head gates; a linear memory with a fixed
 # decay), a selective scan, a clamped gated unit, scaled and soft-capped logits.
 # ---------------------------------------------------------------------------------------------------------
+FEW_ROWS = 16                      # NV_FEW_ROWS
+
+
+def portion_kinds(rows) -> int:
+    """NV_PORTION_* of some sequences from their row counts (host numbers): 1 single tokens, 2 up to FEW_ROWS, 4 more."""
+    kinds = 0
+    for n in rows:
+        kinds |= 0 if n <= 0 else 1 if n == 1 else 2 if n <= FEW_ROWS else 4
+    return kinds
+
+
 def selective_scan(x: torch.Tensor, dt_raw: torch.Tensor, z: torch.Tensor, Bm: torch.Tensor, Cm: torch.Tensor,
                    dt_bias: torch.Tensor, A: torch.Tensor, D_skip: torch.Tensor, state: torch.Tensor, cu_seqlens_q: torch.Tensor,
-                   cu_seqlens_k: torch.Tensor, state_slots: torch.Tensor, max_seqlen_q: int) -> torch.Tensor:
+                   cu_seqlens_k: torch.Tensor, state_slots: torch.Tensor, max_seqlen_q: int, leading_singles: int = 0) -> torch.Tensor:
     """Diagonal recurrence per channel with token-dependent decay and input over a step's rows; state [slots, C, N] float32
-    updated in place; x, dt_raw, z: [T, C]; Bm, Cm: [T, N]; A [C, N] float32 (negative); returns y * silu(z), [T, C]."""
+    updated in place; x, dt_raw, z: [T, C]; Bm, Cm: [T, N]; A [C, N] float32 (negative); returns y * silu(z), [T, C].
+    leading_singles: sequences in front of the batch with exactly one row each."""
     dt = _dt(x, "x")
     T, Cc = x.shape
     N = Bm.shape[1]
@@ -1571,34 +1583,25 @@ def selective_scan(x: torch.Tensor, dt_raw: torch.Tensor, z: torch.Tensor, Bm: t
         return out
     dll = _lib.mixers()
     mq = max(int(max_seqlen_q), 1)
-    need = dll.nv_selective_scan_workspace_bytes(B, Cc, N, mq)
+    lead = B if mq == 1 else int(leading_singles)
+    need = dll.nv_selective_scan_workspace_bytes(B, T, Cc, N, mq, lead)
     ws = _workspace(x.device, need) if need else None
     rc = dll.nv_selective_scan(x.data_ptr(), x.stride(0), dt_raw.data_ptr(), dt_raw.stride(0), z.data_ptr(), z.stride(0),
                                Bm.data_ptr(), Bm.stride(0), Cm.data_ptr(), Cm.stride(0), _f32c(dt_bias, "dt_bias"),
                                _f32c(A, "A"), _f32c(D_skip, "D"), state.data_ptr(), out.data_ptr(), out.stride(0),
-                               cu_seqlens_q.data_ptr(), cu_seqlens_k.data_ptr(), state_slots.data_ptr(), B, Cc, N, mq, dt,
-                               _ptr(ws), ws.numel() if ws is not None else 0, _stream(x))
+                               cu_seqlens_q.data_ptr(), cu_seqlens_k.data_ptr(), state_slots.data_ptr(), B, T, Cc, N, mq,
+                               lead, dt, _ptr(ws), ws.numel() if ws is not None else 0, _stream(x))
     _lib.check(rc, "nv_selective_scan", dll)
     return out
 
 
-FEW_ROWS = 16                      # NV_FEW_ROWS
-
-
-def portion_kinds(rows) -> int:
-    """NV_PORTION_* of a step from its sequences' row counts (host numbers): 1 single tokens, 2 up to FEW_ROWS, 4 more."""
-    kinds = 0
-    for n in rows:
-        kinds |= 0 if n <= 0 else 1 if n == 1 else 2 if n <= FEW_ROWS else 4
-    return kinds
-
-
 def fixed_decay_memory(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor, state: torch.Tensor,
                        cu_seqlens_q: torch.Tensor, cu_seqlens_k: torch.Tensor, state_slots: torch.Tensor, max_seqlen_q: int,
-                       portions: int = 7) -> torch.Tensor:
+                       leading_singles: int = 0, portions: int = 7) -> torch.Tensor:
     """S <- decay_h S + silu(k) silu(v)^T, o = S^T silu(q) over a step's rows; q, k: [T, H, Dk]; v: [T, H, Dv] as projected;
-    decay [H] float32; state [slots, H, Dk, Dv] float32 updated in place; returns o as float32 [T, H * Dv].  portions: the kinds
-    of portions in the step (`portion_kinds`; 7: not known)."""
+    decay [H] float32; state [slots, H, Dk, Dv] float32 updated in place; returns o as float32 [T, H * Dv].
+    leading_singles: sequences in front of the batch with exactly one row each; portions: the kinds of portions behind them
+    (`portion_kinds`; 7: not known)."""
     dt = _dt(q, "q")
     T, H, Dk = q.shape
     Dv = v.shape[2]
@@ -1614,12 +1617,13 @@ def fixed_decay_memory(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay:
         return out
     dll = _lib.mixers()
     mq = max(int(max_seqlen_q), 1)
-    need = dll.nv_fixed_decay_workspace_bytes(B, H, Dk, Dv, mq, dt)
+    lead = B if mq == 1 else int(leading_singles)
+    need = dll.nv_fixed_decay_workspace_bytes(B, T, H, Dk, Dv, mq, lead, dt)
     ws = _workspace(q.device, need) if need else None
     rc = dll.nv_fixed_decay_memory(q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0), k.stride(0), v.stride(0),
                                    _f32c(decay, "decay"), state.data_ptr(), out.data_ptr(), out.stride(0),
-                                   cu_seqlens_q.data_ptr(), cu_seqlens_k.data_ptr(), state_slots.data_ptr(), B, H, Dk, Dv, mq,
-                                   int(portions), dt, _ptr(ws), ws.numel() if ws is not None else 0, _stream(q))
+                                   cu_seqlens_q.data_ptr(), cu_seqlens_k.data_ptr(), state_slots.data_ptr(), B, T, H, Dk, Dv, mq,
+                                   lead, int(portions), dt, _ptr(ws), ws.numel() if ws is not None else 0, _stream(q))
     _lib.check(rc, "nv_fixed_decay_memory", dll)
     return out
 

@@ -56,8 +56,8 @@ class CacheContext:
     # Extension (optional): host copy (numpy int32 [B+1]) of cu_seqlens_q, for layers that lay out their launch per
     # sequence on the host (layers/chunk_attention.py cuts prompt portions into row tiles).
     cu_seqlens_q_host: Optional[object] = None
-    # Extension (optional): which kinds of portions the step holds (`ops.portion_kinds`), for layers with a launch for each
-    # (layers/gated_memory.py).
+    # Extension (optional): which kinds of portions stand behind the leading single rows (`ops.portion_kinds`), for layers with
+    # a launch for each (layers/gated_memory.py).
     portion_kinds: int = 7
 
 

@@ -36,16 +36,22 @@ def dt(request):
 N_Q, N_K, SLOTS = [5, 1, 17, 2, 64, 131, 1], [5, 40, 30, 2, 64, 140, 9], [2, 0, 3, 1, 6, 4, 5]
 
 
-def set_step(n_q, n_k, slots):
+def set_step(n_q, n_k, slots, hints=True):
     ctx, pos = paged_context(n_q, n_k, 8, sum(-(-n // 8) for n in n_k) + 4, 1, DEV, slots=slots)
-    ctx.portion_kinds = nv.ops.portion_kinds(n_q)
+    if hints:                                           # as the runner gives them; without them every launch is prepared for anything
+        ctx.num_leading_decode = next((i for i, n in enumerate(n_q) if n != 1), len(n_q))
+        ctx.portion_kinds = nv.ops.portion_kinds(n_q[ctx.num_leading_decode:])
     nv.set_context(ctx)
     return sum(n_q), pos
 
 
-@pytest.fixture
-def step():
-    yield set_step(N_Q, N_K, SLOTS)
+@pytest.fixture(params=["hints", "no_hints", "singles_first"])
+def step(request):
+    n_q, n_k = N_Q, N_K
+    if request.param == "singles_first":
+        order = sorted(range(len(N_Q)), key=lambda i: N_Q[i] != 1)
+        n_q, n_k = [N_Q[i] for i in order], [N_K[i] for i in order]
+    yield set_step(n_q, n_k, SLOTS, request.param != "no_hints")
     nv.set_context(None)
 
 
@@ -97,7 +103,7 @@ def test_selective_scan(dt, step, C, N):
     assert torch.equal(sa[7], sb[7])                                           # the slot nobody holds
 
 
-@pytest.mark.parametrize("C,N,n_q", [(64, 16, [700]), (48, 4, [1, 1111, 300, 2]), (2048, 16, [513]), (2048, 16, [40] * 70)])
+@pytest.mark.parametrize("C,N,n_q", [(64, 16, [700]), (48, 4, [1, 1111, 300, 2]), (64, 8, [1] * 40 + [900, 3, 1, 650, 17, 1, 800]), (2048, 16, [513]), (2048, 16, [40] * 70)])
 def test_selective_scan_segments_and_many_sequences(dt, C, N, n_q):
     """Long portions of few sequences run in segments; many sequences take eight states per lane."""
     slots = list(range(len(n_q)))[::-1]
@@ -171,7 +177,7 @@ def test_fixed_decay_chunks_round_nothing_but_the_activations():
     assert rel(ya, yb) < 3e-5 and rel(ca["state"], cb["state"]) < 3e-5
 
 
-@pytest.mark.parametrize("H,Dk,Dv,n_q", [(2, 32, 64, [700]), (1, 64, 32, [1, 1111, 300, 2]), (8, 128, 128, [2048])])
+@pytest.mark.parametrize("H,Dk,Dv,n_q", [(2, 32, 64, [700]), (1, 64, 32, [1, 1111, 300, 2]), (2, 32, 32, [1] * 40 + [900, 3, 1, 650, 17, 1, 800]), (8, 128, 128, [2048])])
 def test_fixed_decay_segments(dt, H, Dk, Dv, n_q):
     slots = list(range(len(n_q)))[::-1]
     T, _ = set_step(n_q, [n + 3 * ((i + 1) % 2) for i, n in enumerate(n_q)], slots)

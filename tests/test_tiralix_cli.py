@@ -125,10 +125,12 @@ def test_launch_plans_of_any_size_are_answered():
     """The workspace queries plan a launch on the host: few channels, long portions, many sequences and one."""
     from nanovllm_amd import _lib
     dll = _lib.mixers()
-    for B in (1, 2, 70, 300):
+    for B, rest, lead in ((1, 0, 0), (2, 1, 1), (70, 69, 0), (300, 2000, 250)):
         for mq in (1, 2, 16, 17, 255, 256, 512, 1000, 100000):
+            T = mq + rest
             for C, N in ((1, 1), (7, 3), (24, 6), (100, 256), (20000, 16)):
-                assert 0 <= dll.nv_selective_scan_workspace_bytes(B, C, N, mq) <= 4 * B * 16 * C * (N + 1)
+                assert 0 <= dll.nv_selective_scan_workspace_bytes(B, T, C, N, mq, lead) <= 4 * (2 * 16 * T // mq + 2) * C * (N + 1)
             for H, Dk, Dv in ((1, 1, 1), (3, 5, 65), (64, 128, 256)):
-                assert 0 <= dll.nv_fixed_decay_workspace_bytes(B, H, Dk, Dv, mq, 0) <= 4 * B * 16 * H * Dk * Dv
-                assert dll.nv_fixed_decay_workspace_bytes(B, H, Dk, Dv, mq, 1) == 0        # float32 rows run token by token
+                assert 0 <= dll.nv_fixed_decay_workspace_bytes(B, T, H, Dk, Dv, mq, lead, 0) <= 4 * (2 * 16 * T // mq + 2) * H * Dk * Dv
+                assert dll.nv_fixed_decay_workspace_bytes(B, T, H, Dk, Dv, mq, lead, 1) == 0        # float32 rows run token by token
+    assert dll.nv_selective_scan_workspace_bytes(5, 5, 64, 16, 1, 5) == dll.nv_fixed_decay_workspace_bytes(5, 5, 2, 32, 32, 1, 5, 0) == 0

@@ -71,7 +71,8 @@ def kernel_records(dev):
     for name, n_qs in cases.items():
         note("recurrent kernels, " + name)
         ctx, pos, _ = paged(n_qs, [n + 100 for n in n_qs], bs, dev)
-        ctx.portion_kinds = ops.portion_kinds(n_qs)
+        ctx.num_leading_decode = sum(n == 1 for n in n_qs)                 # (the lists lead with their single tokens)
+        ctx.portion_kinds = ops.portion_kinds(n_qs[ctx.num_leading_decode:])
         T, B = sum(n_qs), len(n_qs)
         nv.set_context(ctx)
         rec = {}
